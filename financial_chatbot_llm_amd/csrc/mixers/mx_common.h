@@ -61,3 +61,14 @@ __device__ __forceinline__ float mx_sigmoid(float x) { return 1.0f / (1.0f + exp
 __device__ __forceinline__ float mx_silu(float x) { return x * mx_sigmoid(x); }
 // softplus without a clamp: log(1 + e^x), evaluated so that neither tail overflows
 __device__ __forceinline__ float mx_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+// tanh with one division and no branch.  |z| < 0.6: the fifth convergent of Lambert's continued fraction
+// z / (1 + z^2 / (3 + z^2 / (5 + ...))), relative error below 1e-8 there; beyond: (1 - e) / (1 + e), e = exp(-2|z|)
+__device__ __forceinline__ float mx_tanh(float z) {
+  const float a = fabsf(z), q = z * z;
+  const bool small = a < 0.6f;
+  const float e = __expf(-2.0f * a);
+  const float num = small ? a * (945.0f + q * (105.0f + q)) : 1.0f - e;
+  const float den = small ? 945.0f + q * (420.0f + 15.0f * q) : 1.0f + e;
+  return copysignf(num / den, z);
+}

@@ -6,8 +6,11 @@
 //         x <- x + sigmoid(gate + gate_bias) * (mult_a * a + mult_b * b)
 //   * RMS norm of a strided row slice (latent norms), optionally in equal groups and with a SiLU
 //     gate applied first (the state-space mixer's output norm);
+//   * elementwise norms D(v) = tanh(alpha v) * w + b around a sublayer, one pass over the stream:
+//         x <- x + D1(y) (or x <- D1(scale * table[id]) at the embedding);  out = D2(x)
 //   * activations: relu^2, and the clamped gated unit g * sigmoid(alpha g) * (u + 1);
-//   * biased top-k routing: softmax scores, choice = score + bias, weights = unbiased scores;
+//   * biased top-k routing: softmax or sigmoid scores, choice = score + bias, weights = unbiased scores,
+//     optionally divided by the sum of the chosen ones and times a constant;
 //   * weighted combine of routed expert rows, identity experts and a shared expert.
 #include "mx_common.h"
 
@@ -93,6 +96,57 @@ __global__ void relu2_kernel(const T* __restrict__ in, long si, T* __restrict__ 
   }
 }
 
+// grid (row groups, column chunks): a thread owns V adjacent columns and walks `rows` rows, its weights in
+// registers.  a null: the first form reads table rows (ids) and REPLACES x; both a and table null: out only.
+template <typename TA, typename TO, int V>
+__global__ void dyn_tanh_kernel(float* __restrict__ x, const TA* __restrict__ a, long sa, const int* __restrict__ ids,
+                                const TA* __restrict__ table, int vocab, float scale, float alpha1,
+                                const float* __restrict__ w1, const float* __restrict__ b1, float alpha2,
+                                const float* __restrict__ w2, const float* __restrict__ b2, TO* __restrict__ out, int W,
+                                int rows, int T) {
+  typedef float vf __attribute__((ext_vector_type(V)));
+  typedef TA va __attribute__((ext_vector_type(V)));
+  typedef TO vo __attribute__((ext_vector_type(V)));
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= W) return;
+  const bool pre = a != nullptr || table != nullptr;
+  vf w1r = {}, b1r = {}, w2r = {}, b2r = {};
+  if (pre) {
+    w1r = *reinterpret_cast<const vf*>(w1 + c);
+    b1r = *reinterpret_cast<const vf*>(b1 + c);
+  }
+  if (out != nullptr) {
+    w2r = *reinterpret_cast<const vf*>(w2 + c);
+    b2r = *reinterpret_cast<const vf*>(b2 + c);
+  }
+  const long t0 = (long)blockIdx.x * rows, t1 = min(t0 + rows, (long)T);
+  for (long t = t0; t < t1; ++t) {
+    float* xr = x + t * W + c;
+    vf v = {};
+    if (a != nullptr) {
+      const va y = *reinterpret_cast<const va*>(a + t * sa + c);
+      v = *reinterpret_cast<const vf*>(xr);
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] += mx_tanh(alpha1 * (float)y[e]) * w1r[e] + b1r[e];
+    } else if (table != nullptr) {
+      int id = ids[t];
+      id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+      const va y = *reinterpret_cast<const va*>(table + (long)id * W + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = mx_tanh(alpha1 * (scale * (float)y[e])) * w1r[e] + b1r[e];
+    } else {
+      v = *reinterpret_cast<const vf*>(xr);
+    }
+    if (pre) *reinterpret_cast<vf*>(xr) = v;
+    if (out != nullptr) {
+      vo o;
+#pragma unroll
+      for (int e = 0; e < V; ++e) o[e] = (TO)(mx_tanh(alpha2 * v[e]) * w2r[e] + b2r[e]);
+      *reinterpret_cast<vo*>(out + t * W + c) = o;
+    }
+  }
+}
+
 // gate and up are column slices (row strides sg / su) of one projection output
 template <typename T>
 __global__ void glu_clamp_kernel(const T* __restrict__ gate, long sg, const T* __restrict__ up, long su,
@@ -106,21 +160,45 @@ __global__ void glu_clamp_kernel(const T* __restrict__ gate, long sg, const T* _
   }
 }
 
-// one wave per token: scores = softmax(z) over all E entries; the `top` largest score + bias are
-// chosen (ties: the lower index), each with its unbiased score as weight.
-__global__ void route_biased_kernel(const float* __restrict__ z, const float* __restrict__ bias, int E, int top,
-                                    float* __restrict__ outw, int* __restrict__ outi, int T) {
+// the same with 16-byte accesses: grid (rows, column chunks), V elements per thread; every row start and the
+// column count are multiples of V elements
+template <typename T, int V>
+__global__ void glu_clamp_vec_kernel(const T* __restrict__ gate, long sg, const T* __restrict__ up, long su, float limit,
+                                     float alpha, T* __restrict__ out, long so, int nv) {
+  typedef T vec __attribute__((ext_vector_type(V)));
+  const long t = blockIdx.x;
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= nv) return;
+  const vec gv = *reinterpret_cast<const vec*>(gate + t * sg + (long)c * V);
+  const vec uv = *reinterpret_cast<const vec*>(up + t * su + (long)c * V);
+  vec o;
+#pragma unroll
+  for (int e = 0; e < V; ++e) {
+    const float g = fminf((float)gv[e], limit);
+    const float u = fminf(fmaxf((float)uv[e], -limit), limit);
+    o[e] = (T)(g * mx_sigmoid(alpha * g) * (u + 1.0f));
+  }
+  *reinterpret_cast<vec*>(out + t * so + (long)c * V) = o;
+}
+
+// one wave per token: scores = softmax(z) over all E entries, or (sigm) sigmoid(z) of each; the `top` largest
+// score + bias are chosen (ties: the lower index), each with its unbiased score as weight -- with renorm divided
+// by the chosen scores' sum (+ 1e-20) -- times wscale.
+__global__ void route_biased_kernel(const float* __restrict__ z, const float* __restrict__ bias, int E, int top, int sigm,
+                                    int renorm, float wscale, float* __restrict__ outw, int* __restrict__ outi, int T) {
   const int t = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
   if (t >= T) return;
   const float* zr = z + (long)t * E;
-  float m = -INFINITY;
-  for (int e = lane; e < E; e += 64) m = fmaxf(m, zr[e]);
-  m = mx_wave_max(m);
-  float s = 0.f;
-  for (int e = lane; e < E; e += 64) s += expf(zr[e] - m);
-  s = mx_wave_sum(s);
-  const float inv = 1.0f / s;
+  float m = -INFINITY, inv = 1.f;
+  if (!sigm) {
+    for (int e = lane; e < E; e += 64) m = fmaxf(m, zr[e]);
+    m = mx_wave_max(m);
+    float s = 0.f;
+    for (int e = lane; e < E; e += 64) s += expf(zr[e] - m);
+    inv = 1.0f / mx_wave_sum(s);
+  }
+  float wsum = 0.f;                                  // lane 0: the chosen scores' sum
   unsigned long long taken_lo = 0, taken_hi = 0;     // this lane's entries already chosen (E <= 64 * 128)
   for (int k = 0; k < top; ++k) {
     float bv = -INFINITY;
@@ -128,7 +206,7 @@ __global__ void route_biased_kernel(const float* __restrict__ z, const float* __
     for (int e = lane, j = 0; e < E; e += 64, ++j) {
       const bool used = j < 64 ? (taken_lo >> j) & 1 : (taken_hi >> (j - 64)) & 1;
       if (used) continue;
-      const float c = expf(zr[e] - m) * inv + (bias != nullptr ? bias[e] : 0.f);
+      const float c = (sigm ? mx_sigmoid(zr[e]) : expf(zr[e] - m) * inv) + (bias != nullptr ? bias[e] : 0.f);
       if (c > bv || (c == bv && e < bi)) {
         bv = c;
         bi = e;
@@ -150,8 +228,14 @@ __global__ void route_biased_kernel(const float* __restrict__ z, const float* __
     if (lane == 0) {
       const int e = bi == 0x7fffffff ? 0 : bi;
       outi[(long)t * top + k] = e;
-      outw[(long)t * top + k] = bi == 0x7fffffff ? 0.f : expf(zr[e] - m) * inv;
+      const float sc = bi == 0x7fffffff ? 0.f : (sigm ? mx_sigmoid(zr[e]) : expf(zr[e] - m) * inv);
+      wsum += sc;
+      outw[(long)t * top + k] = renorm ? sc : sc * wscale;
     }
+  }
+  if (renorm && lane == 0) {
+    const float f = wscale / (wsum + 1e-20f);
+    for (int k = 0; k < top; ++k) outw[(long)t * top + k] *= f;
   }
 }
 
@@ -196,6 +280,32 @@ MX_API int mx_residual_norm(float* x, const void* a, long sa, const void* b, lon
   MX_RETURN_LAUNCH();
 }
 
+// x f32 [T, W].  a given ([T, >= W] slice, row stride sa, type dt_a): x <- x + D1(a); else table given ([vocab, W] of
+// type dt_a, ids [T]): x <- D1(scale * table[id]).  Then, with out ([T, W] of type dt_out): out = D2(x).
+// D(v) = tanh(alpha v) * w + b elementwise, w and b f32 [W].
+MX_API int mx_dyn_tanh(float* x, const void* a, long sa, const int* ids, const void* table, int vocab, float scale,
+                       int dt_a, float alpha1, const float* w1, const float* b1, float alpha2, const float* w2,
+                       const float* b2, void* out, int dt_out, int T, int W, hipStream_t st) {
+  if (T <= 0) return 0;
+  if ((a != nullptr || table != nullptr) && (w1 == nullptr || b1 == nullptr)) return (int)hipErrorInvalidValue;
+  if (out != nullptr && (w2 == nullptr || b2 == nullptr)) return (int)hipErrorInvalidValue;
+  if (table != nullptr && ids == nullptr) return (int)hipErrorInvalidValue;
+  const bool vec = W % 4 == 0 && sa % 4 == 0 && ((size_t)a | (size_t)table) % (dt_a == 1 ? 16 : 8) == 0 &&
+                   ((size_t)x | (size_t)w1 | (size_t)b1 | (size_t)w2 | (size_t)b2) % 16 == 0 &&
+                   (size_t)out % (dt_out == 1 ? 16 : 8) == 0;
+  const int cols = vec ? W / 4 : W;
+  const int nt = cols >= 256 ? 256 : (cols + 63) / 64 * 64;
+  const int rows = T >= 2048 ? 4 : (T >= 1024 ? 2 : 1);
+  dim3 grid((T + rows - 1) / rows, (cols + nt - 1) / nt);
+  if (vec)
+    MX_DISPATCH(dt_a, TA, MX_DISPATCH(dt_out, TO, dyn_tanh_kernel<TA, TO, 4><<<grid, nt, 0, st>>>(
+        x, (const TA*)a, sa, ids, (const TA*)table, vocab, scale, alpha1, w1, b1, alpha2, w2, b2, (TO*)out, W, rows, T)));
+  else
+    MX_DISPATCH(dt_a, TA, MX_DISPATCH(dt_out, TO, dyn_tanh_kernel<TA, TO, 1><<<grid, nt, 0, st>>>(
+        x, (const TA*)a, sa, ids, (const TA*)table, vocab, scale, alpha1, w1, b1, alpha2, w2, b2, (TO*)out, W, rows, T)));
+  MX_RETURN_LAUNCH();
+}
+
 // in [T, groups * n] (row stride si, type dt_in; f32 when dt_in == 1), optional gate of type dt_gate
 MX_API int mx_group_norm(const void* in, long si, int dt_in, const void* gate, long sg, int dt_gate, const float* w,
                          float eps, void* out, long so, int dt_out, int T, int groups, int n, hipStream_t st) {
@@ -219,17 +329,33 @@ MX_API int mx_glu_clamp(const void* gate, long sg, const void* up, long su, floa
                         long so, int dt, int T, int n, hipStream_t st) {
   const long total = (long)T * n;
   if (total <= 0) return 0;
+  const int V = dt == 1 ? 4 : 8;                       // elements per 16 bytes
+  if (n % V == 0 && sg % V == 0 && su % V == 0 && so % V == 0 && ((size_t)gate | (size_t)up | (size_t)out) % 16 == 0 &&
+      (size_t)n / V <= 65535u * 256u) {
+    const int nv = n / V;
+    const int nt = nv >= 256 ? 256 : (nv + 63) / 64 * 64;
+    dim3 grid(T, (nv + nt - 1) / nt);
+    if (dt == 1)
+      glu_clamp_vec_kernel<float, 4><<<grid, nt, 0, st>>>((const float*)gate, sg, (const float*)up, su, limit, alpha,
+                                                          (float*)out, so, nv);
+    else
+      glu_clamp_vec_kernel<bf16, 8><<<grid, nt, 0, st>>>((const bf16*)gate, sg, (const bf16*)up, su, limit, alpha,
+                                                         (bf16*)out, so, nv);
+    MX_RETURN_LAUNCH();
+  }
   const int blocks = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
   MX_DISPATCH(dt, TT, glu_clamp_kernel<TT><<<blocks, 256, 0, st>>>((const TT*)gate, sg, (const TT*)up, su, limit,
                                                                     alpha, (TT*)out, so, n, total));
   MX_RETURN_LAUNCH();
 }
 
-MX_API int mx_route_biased(const float* z, const float* bias, int E, int top, float* outw, int* outi, int T,
-                           hipStream_t st) {
+// sigm != 0: sigmoid scores instead of a softmax over the entries; renorm != 0: weights divided by the sum of the
+// chosen scores (+ 1e-20); wscale: constant on the weights
+MX_API int mx_route_biased(const float* z, const float* bias, int E, int top, int sigm, int renorm, float wscale,
+                           float* outw, int* outi, int T, hipStream_t st) {
   if (T <= 0) return 0;
   if (E > 64 * 128 || top > E) return (int)hipErrorInvalidValue;
-  route_biased_kernel<<<(T + 3) / 4, 256, 0, st>>>(z, bias, E, top, outw, outi, T);
+  route_biased_kernel<<<(T + 3) / 4, 256, 0, st>>>(z, bias, E, top, sigm, renorm, wscale, outw, outi, T);
   MX_RETURN_LAUNCH();
 }
 

@@ -12,6 +12,9 @@
 //     window's own tiles;
 //   * sigmoid weights: with a per-head bias array the weight of a visible key is
 //     sigmoid(score + head_bias[h]) and the weights are NOT normalised over the keys (no softmax).
+// Further options, each an optional argument: a distance bias (slope[h] * (p - j) is taken off the scaled
+// score), a sink (the softmax denominator of head h also holds exp(sink[h]), once, with no key and no value)
+// and a gate per output element instead of per head (out[t, h, :] *= sigmoid(gate[t, h*P + :])).
 //
 //   mx_qk_norm_write   RMS norm over the WHOLE query projection and over the whole key projection
 //                      (all heads at once, plain weights), cache write of [normed k | v].
@@ -34,6 +37,15 @@ __device__ __forceinline__ int first_key(int p, int window, int chunked) {
 // the window's first tile, then the tiles first_tile .. last_tile.  Walk index -> first key of the tile.
 __device__ __forceinline__ int walk_k0(int ti, int nsink, int first_tile, int KT) {
   return (ti < nsink ? ti : first_tile + ti - nsink) * KT;
+}
+
+// factor on the accumulated values of a softmax with running maximum m and sum l: 1 / l, or with a sink
+// exp(m) / (exp(m) l + exp(sink)) evaluated from the larger exponent down
+__device__ __forceinline__ float softmax_scale(float m, float l, const float* sink, int h) {
+  if (sink == nullptr) return 1.0f / l;
+  const float sk = sink[h], M = fmaxf(m, sk);
+  const float f = expf(m - M);
+  return f / (l * f + expf(sk - M));
 }
 
 // one block per token
@@ -86,8 +98,9 @@ template <typename T>
 __global__ void __launch_bounds__(WA_WAVES * 64)
 window_attend_kernel(const T* __restrict__ q, long sq, const T* __restrict__ cache, const int* __restrict__ cu,
                      const int* __restrict__ pos, const int* __restrict__ bt, int btw, const T* __restrict__ gate,
-                     long sgate, int window, int chunked, int keep, const float* __restrict__ hbias, float scale,
-                     T* __restrict__ out, int H, int G, int D, int P, int QT, int HB, int KT, int ldk, int ldv) {
+                     long sgate, int gate_elem, int window, int chunked, int keep, const float* __restrict__ hbias,
+                     const float* __restrict__ slope, const float* __restrict__ sink, float scale, T* __restrict__ out,
+                     int H, int G, int D, int P, int QT, int HB, int KT, int ldk, int ldv) {
   extern __shared__ __align__(16) unsigned char smem[];
   T* ktile = reinterpret_cast<T*>(smem);                                  // [KT][ldk]
   T* vtile = ktile + (size_t)KT * ldk;                                    // [KT][ldv]
@@ -163,6 +176,7 @@ window_attend_kernel(const T* __restrict__ q, long sq, const T* __restrict__ cac
         float a = 0.f;
         for (int d = 0; d < D; ++d) a += myq[d] * ldf(kr + d);
         sc = a * scale;
+        if (slope != nullptr) sc -= slope[h] * (float)(p - j);
       }
       float corr = 1.f, pj;
       if (hbias != nullptr) {                              // independent sigmoid weights, no running statistics
@@ -197,12 +211,16 @@ window_attend_kernel(const T* __restrict__ q, long sq, const T* __restrict__ cac
     const int tq = item / nh, hh = item - tq * nh;
     const long row = r0 + t0 + tq;
     const int h = h0 + hh;
-    float gs = hbias != nullptr ? 1.0f : 1.0f / l[ii];
-    if (gate != nullptr) gs *= mx_sigmoid(ldf(gate + row * sgate + h));
+    float gs = hbias != nullptr ? 1.0f : softmax_scale(m[ii], l[ii], sink, h);
+    if (gate != nullptr && !gate_elem) gs *= mx_sigmoid(ldf(gate + row * sgate + h));
 #pragma unroll
     for (int c = 0; c < WA_CPL; ++c) {
       const int d = lane + 64 * c;
-      if (d < P) stf(out + (row * H + h) * P + d, acc[ii][c] * gs);
+      if (d < P) {
+        float v = acc[ii][c] * gs;
+        if (gate_elem) v *= mx_sigmoid(ldf(gate + row * sgate + (long)h * P + d));
+        stf(out + (row * H + h) * P + d, v);
+      }
     }
   }
 }
@@ -230,8 +248,9 @@ template <int KSM, int NTM>         // up to 32*KSM key dims, 16*NTM value dims
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2)))
 window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __restrict__ cache,
                           const int* __restrict__ cu, const int* __restrict__ pos, const int* __restrict__ bt, int btw,
-                          const bf16* __restrict__ gate, long sgate, int window, int chunked, int keep,
-                          const float* __restrict__ hbias, float scale, bf16* __restrict__ out, int H, int G, int D,
+                          const bf16* __restrict__ gate, long sgate, int gate_elem, int window, int chunked, int keep,
+                          const float* __restrict__ hbias, const float* __restrict__ slope,
+                          const float* __restrict__ sink, float scale, bf16* __restrict__ out, int H, int G, int D,
                           int P, int QT, int HB, int nsplit, float* __restrict__ ws) {
   extern __shared__ __align__(16) unsigned char smem[];
   const int KS = (D + 31) / 32, NT = (P + 15) / 16;
@@ -267,6 +286,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
   const bool wave_live = 16 * wave < nq * nh;
   const bool sigm = hbias != nullptr;
   const float hb = (sigm && qok) ? hbias[h] : 0.f;
+  const float slp = (slope != nullptr && qok) ? slope[h] : 0.f;     // distance bias: score + slp * (j - p)
 
   bf16x8 qf[KSM];
 #pragma unroll
@@ -367,6 +387,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
     f32x4 st[2];
     float sc[2][4];
     float tmax = -INFINITY;
+    const float dist0 = (float)(k0 + 4 * g - pq);          // j - p of this lane's first key (exact in f32)
 #pragma unroll
     for (int kh = 0; kh < 2; ++kh) {
       st[kh] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -378,7 +399,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
       for (int i = 0; i < 4; ++i) {
         const int j = k0 + 16 * kh + 4 * g + i;
         const bool vis = j <= pq && (j >= pq_lo || j < keep);
-        sc[kh][i] = vis ? st[kh][i] * scale : -INFINITY;
+        sc[kh][i] = vis ? st[kh][i] * scale + slp * (dist0 + (float)(16 * kh + i)) : -INFINITY;
         tmax = fmaxf(tmax, sc[kh][i]);
       }
     }
@@ -438,16 +459,36 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
     }
     return;
   }
-  float gsc = sigm ? 1.0f : 1.0f / l;
-  if (gate != nullptr) gsc *= mx_sigmoid((float)gate[row * sgate + h]);
+  float gsc = sigm ? 1.0f : softmax_scale(m, l, sink, h);
+  if (gate != nullptr && !gate_elem) gsc *= mx_sigmoid((float)gate[row * sgate + h]);
   bf16* dst = out + (row * H + h) * P;
+  const bf16* ge = gate_elem ? gate + row * sgate + (long)h * P : nullptr;
+  if ((P & 3) == 0 && (gate_elem == 0 || gate_elem == 2)) {      // 8-byte accesses (2: the gate's rows allow them)
+#pragma unroll
+    for (int nt = 0; nt < NTM; ++nt) {
+      const int r = 16 * nt + 4 * g;
+      if (nt < NT && r < P) {
+        f32x4 v = o[nt] * gsc;
+        if (ge != nullptr) {
+          const bf16x4 gv = *reinterpret_cast<const bf16x4*>(ge + r);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) v[i] *= mx_sigmoid((float)gv[i]);
+        }
+        bf16x4 w4;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) w4[i] = (bf16)v[i];
+        *reinterpret_cast<bf16x4*>(dst + r) = w4;
+      }
+    }
+    return;
+  }
 #pragma unroll
   for (int nt = 0; nt < NTM; ++nt) {
     if (nt < NT) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int r = 16 * nt + 4 * g + i;
-        if (r < P) dst[r] = (bf16)(o[nt][i] * gsc);
+        if (r < P) dst[r] = (bf16)(o[nt][i] * gsc * (ge != nullptr ? mx_sigmoid((float)ge[r]) : 1.0f));
       }
     }
   }
@@ -456,35 +497,37 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
 // grid (rows, H): combine the nsplit parts of one (row, head)
 // (sigm: the parts are plain sums of independently weighted values)
 __global__ void window_merge_kernel(const float* __restrict__ ws, const bf16* __restrict__ gate, long sgate,
-                                    bf16* __restrict__ out, int H, int P, int nsplit, int sigm) {
+                                    int gate_elem, const float* __restrict__ sink, bf16* __restrict__ out, int H, int P,
+                                    int nsplit, int sigm) {
   const long row = blockIdx.x;
   const int h = blockIdx.y;
   const float* w = ws + (row * H + h) * nsplit * (long)(P + 2);
+  const bf16* ge = gate_elem ? gate + row * sgate + (long)h * P : nullptr;
   if (sigm) {
-    const float gs = gate != nullptr ? mx_sigmoid((float)gate[row * sgate + h]) : 1.0f;
+    const float gs = gate != nullptr && !gate_elem ? mx_sigmoid((float)gate[row * sgate + h]) : 1.0f;
     for (int r = threadIdx.x; r < P; r += blockDim.x) {
       float a = 0.f;
       for (int i = 0; i < nsplit; ++i) a += w[i * (P + 2) + r];
-      out[(row * H + h) * P + r] = (bf16)(a * gs);
+      out[(row * H + h) * P + r] = (bf16)(a * gs * (ge != nullptr ? mx_sigmoid((float)ge[r]) : 1.0f));
     }
     return;
   }
-  float M = -INFINITY;
+  float M = sink != nullptr ? sink[h] : -INFINITY;
   for (int i = 0; i < nsplit; ++i) M = fmaxf(M, w[i * (P + 2) + P]);
-  float L = 0.f;
+  float L = sink != nullptr ? expf(sink[h] - M) : 0.f;      // the sink counts once, not once per part
   for (int i = 0; i < nsplit; ++i) {
     const float mi = w[i * (P + 2) + P];
     if (mi != -INFINITY) L += w[i * (P + 2) + P + 1] * expf(mi - M);
   }
   float gsc = 1.0f / L;
-  if (gate != nullptr) gsc *= mx_sigmoid((float)gate[row * sgate + h]);
+  if (gate != nullptr && !gate_elem) gsc *= mx_sigmoid((float)gate[row * sgate + h]);
   for (int r = threadIdx.x; r < P; r += blockDim.x) {
     float a = 0.f;
     for (int i = 0; i < nsplit; ++i) {
       const float mi = w[i * (P + 2) + P];
       if (mi != -INFINITY) a += w[i * (P + 2) + r] * expf(mi - M);
     }
-    out[(row * H + h) * P + r] = (bf16)(a * gsc);
+    out[(row * H + h) * P + r] = (bf16)(a * gsc * (ge != nullptr ? mx_sigmoid((float)ge[r]) : 1.0f));
   }
 }
 
@@ -518,14 +561,20 @@ MX_API int mx_qk_norm_write(const void* q, long sq, const void* k, long sk, cons
 // chunked != 0: `window` is the block size of the chunked mask instead of a sliding window's length.
 // keep > 0: the first `keep` keys of the sequence stay visible beyond the window.  head_bias (f32 [H], or
 // null): sigmoid weights sigmoid(score + head_bias[h]) without normalisation instead of a softmax.
+// slope (f32 [H], or null): score - slope[h] * (p - j).  sink (f32 [H], or null; softmax only): exp(sink[h]) in
+// the denominator.  gate_elem != 0: the gate is a [T, >= H*P] slice, one value per output element.
 // nsplit > 1 with a workspace ws (f32 [T, H, nsplit, P + 2]) and single-row segments: the key range of
 // each row is walked by nsplit blocks and merged (bf16 matrix-core form only; ignored otherwise).
 MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int* cu, const int* pos, const int* bt,
-                            int btw, const void* gate, long sgate, int window, int chunked, int keep,
-                            const float* head_bias, float scale, void* out, int dt, int S, int max_len, int H, int G,
+                            int btw, const void* gate, long sgate, int gate_elem, int window, int chunked, int keep,
+                            const float* head_bias, const float* slope, const float* sink, float scale, void* out, int dt, int S, int max_len, int H, int G,
                             int D, int P, int nsplit, float* ws, hipStream_t st) {
   if (S <= 0 || max_len <= 0) return 0;
-  if (P > 64 * WA_CPL || G < 1 || H % G || window < 1 || keep < 0) return (int)hipErrorInvalidValue;
+  if (P > 64 * WA_CPL || G < 1 || H % G || window < 1 || keep < 0 ||
+      (gate_elem && gate == nullptr) || (sink != nullptr && head_bias != nullptr))
+    return (int)hipErrorInvalidValue;
+  // 2: gate rows that 8-byte accesses may read (bf16)
+  const int ge = !gate_elem ? 0 : (P % 4 == 0 && sgate % 4 == 0 && (size_t)gate % 8 == 0 ? 2 : 1);
   const int rep = H / G;
   if (dt == 0 && D <= 256 && P <= 256 && wa_use_mfma()) {
     // matrix-core form: 64 (row, head) pairs of one key/value head per block
@@ -537,16 +586,16 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
     dim3 grid(nsplit > 1 ? nsplit : (max_len + QT - 1) / QT, G * ((rep + HB - 1) / HB), S);
     if (D <= 128 && P <= 128)
       window_attend_mfma_kernel<4, 8><<<grid, 256, lds, st>>>(
-          (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, window, chunked, keep,
-          head_bias, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
+          (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked,
+          keep, head_bias, slope, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
     else
       window_attend_mfma_kernel<8, 16><<<grid, 256, lds, st>>>(
-          (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, window, chunked, keep,
-          head_bias, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
+          (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked,
+          keep, head_bias, slope, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
     if (nsplit > 1) {
       dim3 g2(S, H);           // single-row segments: row index == segment index
-      window_merge_kernel<<<g2, P >= 128 ? 128 : 64, 0, st>>>(ws, (const bf16*)gate, sgate, (bf16*)out, H, P, nsplit,
-                                                              head_bias != nullptr ? 1 : 0);
+      window_merge_kernel<<<g2, P >= 128 ? 128 : 64, 0, st>>>(ws, (const bf16*)gate, sgate, ge, sink, (bf16*)out, H, P,
+                                                              nsplit, head_bias != nullptr ? 1 : 0);
     }
     MX_RETURN_LAUNCH();
   }
@@ -570,7 +619,7 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
   if (lds > 64 * 1024) return (int)hipErrorInvalidValue;
   dim3 grid((max_len + QT - 1) / QT, G * ((rep + HB - 1) / HB), S);
   MX_DISPATCH(dt, TT, window_attend_kernel<TT><<<grid, WA_WAVES * 64, lds, st>>>(
-      (const TT*)q, sq, (const TT*)cache, cu, pos, bt, btw, (const TT*)gate, sgate, window, chunked, keep, head_bias,
-      scale, (TT*)out, H, G, D, P, QT, HB, KT, ldk, ldv));
+      (const TT*)q, sq, (const TT*)cache, cu, pos, bt, btw, (const TT*)gate, sgate, ge, window, chunked, keep, head_bias,
+      slope, sink, scale, (TT*)out, H, G, D, P, QT, HB, KT, ldk, ldv));
   MX_RETURN_LAUNCH();
 }

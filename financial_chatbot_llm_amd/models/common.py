@@ -72,7 +72,9 @@ class HybridCache:
     * ``("state", taps, channels, heads, vdim, state)`` -> ``("state", conv, ssm)``, f32 conv
       [slots, taps - 1, channels] and ssm [slots, heads, vdim, state];
     * ``("slots", {name: shape})`` -> ``("slots", {name: f32 [slots, *shape]})``;
-    * ``("pair", spec_a, spec_b)`` -> ``("pair", entry_a, entry_b)`` (two mixers side by side).
+    * ``("pair", spec_a, spec_b)`` -> ``("pair", entry_a, entry_b)`` (two mixers side by side, or a mixer with
+      cache rows and slot state);
+    * ``("none",)`` -> ``("none",)``: nothing of its own (a layer that reads another layer's rows).
 
     ``slot_arrays`` ({name: (dtype, shape)}) are per-slot records of the model as a whole
     (``model[name]``: [slots, *shape]), e.g. the last token of each sequence.  Pages and slots are

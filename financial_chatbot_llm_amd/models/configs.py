@@ -15,7 +15,7 @@ from typing import Dict, Optional
 @dataclass(frozen=True)
 class ModelConfig:
     name: str
-    arch: str                       # "llama" | "mixtral" | "bert" | "gezavik" | "sigudra" | "tukedra" | "purozen"
+    arch: str                       # "llama" | "mixtral" | "bert" | "gezavik" | "sigudra" | "tukedra" | "purozen" | "fanotar"
     vocab_size: int
     hidden_size: int
     num_layers: int
@@ -86,6 +86,7 @@ def _register_layered() -> None:
     from .sigudra import example_config as sigudra_config
     from .tukedra import example_config as tukedra_config
     from .purozen import example_config as purozen_config
+    from .fanotar import example_config as fanotar_config
     for name, kw in (("gezavik-tiny", dict(width=192, vocab=1024, heads=3, pattern="amAm")),
                      ("gezavik-1b", dict(width=2048, vocab=32768, heads=16, pattern="aMmAmMaM" * 2, scale_up=True))):
         REGISTRY[name] = layered_config(example_config(**kw), name)
@@ -98,10 +99,13 @@ def _register_layered() -> None:
     for name, kw in (("purozen-tiny", dict(width=160, vocab=896, pattern="paAl")),
                      ("purozen-1b", dict(width=2048, vocab=32768, pattern="paalpaal" * 2, scale_up=True))):
         REGISTRY[name] = layered_config(purozen_config(**kw), name)
+    for name, kw in (("fanotar-tiny", dict(width=160, vocab=704, pattern="AEkK")),
+                     ("fanotar-1b", dict(width=2048, vocab=32768, pattern="AEAKAEkK" * 2, scale_up=True))):
+        REGISTRY[name] = layered_config(fanotar_config(**kw), name)
 
 
 def get_model_config(name: str) -> ModelConfig:
-    if name.startswith(("gezavik-", "sigudra-", "tukedra-", "purozen-")) and name not in REGISTRY:
+    if name.startswith(("gezavik-", "sigudra-", "tukedra-", "purozen-", "fanotar-")) and name not in REGISTRY:
         _register_layered()
     if name in REGISTRY:
         return REGISTRY[name]
@@ -136,7 +140,7 @@ def from_hf(path: str, name: Optional[str] = None) -> ModelConfig:
         top_k_experts=c.get("num_experts_per_tok", 0), bos_token_id=c.get("bos_token_id", 1), eos_token_ids=eos)
 
 
-LAYERED_ARCHS = ("gezavik", "sigudra", "tukedra", "purozen")
+LAYERED_ARCHS = ("gezavik", "sigudra", "tukedra", "purozen", "fanotar")
 
 
 def layered_config(c: Dict, name: Optional[str] = None) -> ModelConfig:

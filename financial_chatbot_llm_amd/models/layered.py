@@ -1,4 +1,5 @@
-"""Common part of the layered decoders (:mod:`.gezavik`, :mod:`.sigudra`, :mod:`.tukedra`, :mod:`.purozen`): a ``config.json`` lists the
+"""Common part of the layered decoders (:mod:`.gezavik`, :mod:`.sigudra`, :mod:`.tukedra`, :mod:`.purozen`,
+:mod:`.fanotar`): a ``config.json`` lists the
 layers, each with one sequence mixer of :mod:`.mixers` and optionally one feed-forward; the residual
 stream is f32 whatever the activation dtype; the checkpoint is the model directory itself (tensors
 ``embed``, ``l<i>.<norm>``, ``l<i>.mix.<name>``, ``l<i>.mlp.<name>``, ``final.norm``, ``head``; linear
@@ -106,8 +107,12 @@ class LayeredDecoder:
             return (1.0 + 0.3 * randn()) / shape[0]
         if ".hc" in name and leaf == "mix":      # stream mixing: near the identity
             return torch.eye(shape[0], device=device) + 0.15 * randn()
-        if leaf in ("norm1", "norm2", "norm", "out") and len(shape) == 1:
+        if leaf in ("norm1", "norm2", "norm1b", "norm2b", "norm", "out") and len(shape) == 1:
             return 1.0 + 0.1 * randn()
+        if leaf == "alpha":        # elementwise norm: mostly the linear part of the tanh
+            return 0.4 + 0.4 * rand()
+        if leaf == "sink":
+            return randn()
         if leaf == "A_log":
             return torch.log(1.0 + 7.0 * rand())
         if leaf == "dt_bias":      # softplus^-1 of step sizes in [0.01, 0.2]

@@ -37,8 +37,12 @@ normed input ``h`` and return a sublayer output, with their sizes and constants 
 * :class:`DenseFF` -- up, activation, down; optionally gated (act(gate) * up).
 * :class:`TopSoftmaxRoutedFF` -- mixture of plain relu^2 experts, softmax over the chosen logits, plus a
   shared expert.
-* :class:`RoutedFF` -- mixture of clamped gated experts with biased top-k choice, identity experts
-  and an always-on shared expert.
+* :class:`ConvAttentionMixer` -- softmax attention whose projected q, k and v pass a short causal convolution;
+  per-head RMS norms with a weight, a query temperature that grows with the position, a distance bias per head,
+  a sliding window, a sink in the softmax denominator, an elementwise output gate; a layer may use an earlier
+  layer's keys and values instead of its own.
+* :class:`RoutedFF` -- mixture of clamped gated experts with biased top-k choice (softmax or sigmoid scores,
+  optionally renormalised and scaled weights), identity experts and an always-on shared expert.
 * :class:`InputScaledRoutedFF` -- mixture of gated experts chosen by independent sigmoid scores, the
   score multiplying the expert's input.
 
@@ -70,6 +74,12 @@ DENSE_MAX_PAIRS = 512
 
 def _capturing(t: torch.Tensor) -> bool:
     return t.is_cuda and torch.cuda.is_current_stream_capturing()
+
+
+def _expert_stack(ws, dtype) -> torch.Tensor:
+    """Expert matrices [out, in] as one batched right operand [E, in, out], contiguous: batched bf16 products take
+    no transposed view."""
+    return torch.stack([w.t() for w in ws]).to(dtype).contiguous()
 
 
 class Mamba2Mixer:
@@ -181,12 +191,14 @@ class LatentAttentionMixer:
 
 class DenseFF:
     """W_down act(W_up h), ``act`` = "relu2" (the square of relu) | gelu_tanh | silu; or, ``gated``,
-    W_down (act(W_gate h) * (W_up h)) with ``act`` in silu | gelu_tanh."""
+    W_down (act(W_gate h) * (W_up h)) with ``act`` in silu | gelu_tanh, or with ``act`` = "clamped" the unit
+    g * sigmoid(alpha g) * (u + 1) of g = min(W_gate h, limit), u = clamp(W_up h, +-limit) (the spec's ``limit``)."""
 
-    def __init__(self, spec: Dict, width: int, act: str = "relu2", gated: bool = False):
+    def __init__(self, spec: Dict, width: int, act: str = "relu2", gated: bool = False, alpha: float = 1.702):
         self.ff, self.width, self.act, self.gated = int(spec["ff"]), width, act, gated
         self.in_rows = self.ff * (2 if gated else 1)
-        if act not in (("silu", "gelu_tanh") if gated else ("relu2", "silu", "gelu_tanh")):
+        self.alpha, self.limit = alpha, float(spec["limit"]) if act == "clamped" else 0.0
+        if act not in (("silu", "gelu_tanh", "clamped") if gated else ("relu2", "silu", "gelu_tanh")):
             raise ValueError(f"unknown activation {act!r} for a {'gated' if gated else 'plain'} feed-forward")
 
     def shapes(self) -> Dict[str, tuple]:
@@ -206,7 +218,10 @@ class DenseFF:
 
     def forward(self, h: torch.Tensor, proj: torch.Tensor, x32: Optional[torch.Tensor] = None) -> torch.Tensor:
         if self.gated:
-            return F.linear(mx.glu_act(proj[:, :self.ff], proj[:, self.ff:2 * self.ff], self.act), self.down)
+            gate, up = proj[:, :self.ff], proj[:, self.ff:2 * self.ff]
+            if self.act == "clamped":
+                return F.linear(mx.glu_clamp(gate, up, self.limit, self.alpha), self.down)
+            return F.linear(mx.glu_act(gate, up, self.act), self.down)
         up = proj[:, :self.ff]
         return F.linear(mx.relu2(up) if self.act == "relu2" else mx.glu_act(up, None, self.act), self.down)
 
@@ -215,12 +230,14 @@ class RoutedFF:
     """Mixture of ``experts`` clamped gated feed-forwards, ``top`` per token.
 
     Router logits z = W_r h in f32; scores s = softmax(z) over the experts and the ``identity``
-    experts that follow them; the ``top`` largest s + correction are chosen and weighted by s itself.
-    An identity expert returns its input.  Expert: g = min(W_g h, limit), u = clamp(W_u h, +-limit),
+    experts that follow them, or (``score="sigmoid"``) each expert's own sigmoid(z); the ``top`` largest
+    s + correction are chosen and weighted by s itself -- with ``renorm`` divided by the chosen scores' sum --
+    times the router's ``scale`` (default 1).  An identity expert returns its input.  Expert: g = min(W_g h, limit), u = clamp(W_u h, +-limit),
     W_d (g * sigmoid(alpha g) * (u + 1)).  A shared expert of the same form runs for every token."""
 
-    def __init__(self, spec: Dict, width: int, alpha: float = 1.702):
+    def __init__(self, spec: Dict, width: int, alpha: float = 1.702, score: str = "softmax", renorm: bool = False):
         r = spec["router"]
+        self.score, self.renorm, self.w_scale = score, renorm, float(r.get("scale", 1.0))
         self.E, self.I, self.top = int(r["experts"]), int(r.get("identity", 0)), int(r["top"])
         self.F = int(spec["expert"]["ff"])
         self.limit = float(spec["expert"]["limit"])
@@ -229,6 +246,8 @@ class RoutedFF:
         self.limit_s = float(sh["limit"]) if sh else 0.0
         self.alpha, self.width = alpha, width
         self.in_rows = 2 * self.Fs                                            # shared gate | up
+        if not 1 <= self.top <= self.E + self.I:
+            raise ValueError("routed feed-forward: 1 <= top <= experts")
 
     def shapes(self) -> Dict[str, tuple]:
         s = {"router": (self.E + self.I, self.width), "correction": (self.E + self.I,)}
@@ -243,8 +262,8 @@ class RoutedFF:
     def load(self, get: Getter, dtype) -> Optional[torch.Tensor]:
         self.router = get("router").float().contiguous()
         self.correction = get("correction").float().contiguous()
-        self.w13 = torch.stack([torch.cat([get(f"e{e}.gate"), get(f"e{e}.up")], 0) for e in range(self.E)]).to(dtype)
-        self.w2 = torch.stack([get(f"e{e}.down") for e in range(self.E)]).to(dtype).contiguous()
+        self.w13 = _expert_stack([torch.cat([get(f"e{e}.gate"), get(f"e{e}.up")], 0) for e in range(self.E)], dtype)
+        self.w2 = _expert_stack([get(f"e{e}.down") for e in range(self.E)], dtype)
         if not self.Fs:
             return None
         self.down_s = get("shared.down").to(dtype).contiguous()
@@ -261,24 +280,28 @@ class RoutedFF:
         if self.Fs:
             shared = F.linear(mx.glu_clamp(proj[:, :self.Fs], proj[:, self.Fs:2 * self.Fs], self.limit_s, self.alpha),
                               self.down_s)
-        wts, idx = mx.route_biased(F.linear(h.float(), self.router), self.correction, top)
+        wts, idx = mx.route_biased(F.linear(h.float(), self.router), self.correction, top, self.score, self.renorm,
+                                   self.w_scale)
         if T * top <= DENSE_MAX_PAIRS or _capturing(h):
-            gu = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w13.transpose(1, 2)).view(E * T, 2 * Fe)
+            gu = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w13).view(E * T, 2 * Fe)
             act = mx.glu_clamp(gu[:, :Fe], gu[:, Fe:], self.limit, self.alpha)
-            ys = torch.bmm(act.view(E, T, Fe), self.w2.transpose(1, 2)).view(E * T, W)
+            ys = torch.bmm(act.view(E, T, Fe), self.w2).view(E * T, W)
             rows = torch.arange(T, dtype=torch.int32, device=h.device)[:, None]
             pos = (idx.clamp(max=E - 1) * T + rows).to(torch.int32)
             return mx.moe_combine(ys, pos, idx, wts, h, shared, E)
         flat = idx.reshape(-1).long()
         order = torch.argsort(flat, stable=True)
         offs = [0] + torch.bincount(flat, minlength=E + self.I).cumsum(0).tolist()     # host read of the buckets
-        xs = h.index_select(0, order // top)
-        ys = torch.empty((T * top, W), dtype=h.dtype, device=h.device)
-        for e in range(E):
-            a, b = offs[e], offs[e + 1]
-            if b > a:
-                gu = F.linear(xs[a:b], self.w13[e])
-                torch.mm(mx.glu_clamp(gu[:, :Fe], gu[:, Fe:], self.limit, self.alpha), self.w2[e].t(), out=ys[a:b])
+        n = offs[E]                                          # rows of real experts (identity experts sort behind them)
+        xs = h.index_select(0, order[:n] // top)
+        live = [(e, offs[e], offs[e + 1]) for e in range(E) if offs[e + 1] > offs[e]]
+        gu = torch.empty((n, 2 * Fe), dtype=h.dtype, device=h.device)
+        for e, a, b in live:
+            torch.mm(xs[a:b], self.w13[e], out=gu[a:b])
+        act = mx.glu_clamp(gu[:, :Fe], gu[:, Fe:], self.limit, self.alpha)             # one launch over all buckets
+        ys = torch.empty((max(n, 1), W), dtype=h.dtype, device=h.device)
+        for e, a, b in live:
+            torch.mm(act[a:b], self.w2[e], out=ys[a:b])
         pos = torch.empty_like(order)
         pos[order] = torch.arange(order.numel(), device=order.device)
         return mx.moe_combine(ys, pos.view(T, top).to(torch.int32), idx, wts, h, shared, E)
@@ -311,8 +334,8 @@ class InputScaledRoutedFF:
 
     def load(self, get: Getter, dtype) -> Optional[torch.Tensor]:
         self.router = get("router").float().contiguous()
-        self.w13 = torch.stack([torch.cat([get(f"e{e}.gate"), get(f"e{e}.up")], 0) for e in range(self.E)]).to(dtype)
-        self.w2 = torch.stack([get(f"e{e}.down") for e in range(self.E)]).to(dtype).contiguous()
+        self.w13 = _expert_stack([torch.cat([get(f"e{e}.gate"), get(f"e{e}.up")], 0) for e in range(self.E)], dtype)
+        self.w2 = _expert_stack([get(f"e{e}.down") for e in range(self.E)], dtype)
         return None
 
     def num_bytes(self) -> int:
@@ -330,9 +353,9 @@ class InputScaledRoutedFF:
             rows = torch.arange(T, device=h.device)[:, None]
             pos = idx.long() * T + rows
             scale = torch.zeros(E * T, dtype=torch.float32, device=h.device).scatter_(0, pos.reshape(-1), wts.reshape(-1))
-            gu = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w13.transpose(1, 2)).view(E * T, 2 * Fe)
+            gu = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w13).view(E * T, 2 * Fe)
             act = mx.glu_act(gu[:, :Fe], gu[:, Fe:], self.act, scale)
-            ys = torch.bmm(act.view(E, T, Fe), self.w2.transpose(1, 2)).view(E * T, W)
+            ys = torch.bmm(act.view(E, T, Fe), self.w2).view(E * T, W)
             return mx.moe_combine(ys, pos.to(torch.int32), idx, ones, h, None, E)
         flat = idx.reshape(-1).long()
         order = torch.argsort(flat, stable=True)
@@ -343,11 +366,11 @@ class InputScaledRoutedFF:
         gu = torch.empty((T * top, 2 * Fe), dtype=h.dtype, device=h.device)
         live = [(e, offs[e], offs[e + 1]) for e in range(E) if offs[e + 1] > offs[e]]
         for e, a, b in live:
-            torch.mm(xs[a:b], self.w13[e].t(), out=gu[a:b])
+            torch.mm(xs[a:b], self.w13[e], out=gu[a:b])
         act = mx.glu_act(gu[:, :Fe], gu[:, Fe:], self.act, sc)
         ys = torch.empty((T * top, W), dtype=h.dtype, device=h.device)
         for e, a, b in live:
-            torch.mm(act[a:b], self.w2[e].t(), out=ys[a:b])
+            torch.mm(act[a:b], self.w2[e], out=ys[a:b])
         pos = torch.empty_like(order)
         pos[order] = torch.arange(order.numel(), device=order.device)
         return mx.moe_combine(ys, pos.view(T, top).to(torch.int32), idx, ones, h, None, E)
@@ -380,8 +403,8 @@ class TopSoftmaxRoutedFF:
 
     def load(self, get: Getter, dtype) -> Optional[torch.Tensor]:
         self.router = get("router").float().contiguous()
-        self.w1 = torch.stack([get(f"e{e}.up") for e in range(self.E)]).to(dtype).contiguous()        # [E, F, W]
-        self.w2 = torch.stack([get(f"e{e}.down") for e in range(self.E)]).to(dtype).contiguous()      # [E, W, F]
+        self.w1 = _expert_stack([get(f"e{e}.up") for e in range(self.E)], dtype)              # [E, W, F]
+        self.w2 = _expert_stack([get(f"e{e}.down") for e in range(self.E)], dtype)            # [E, F, W]
         if not self.Fs:
             return None
         self.down_s = get("shared.down").to(dtype).contiguous()
@@ -397,8 +420,8 @@ class TopSoftmaxRoutedFF:
         shared = F.linear(mx.relu2(proj[:, :self.Fs]), self.down_s) if self.Fs else None
         wts, idx = mx.route_scores(F.linear(x32 if x32 is not None else h.float(), self.router), top, "softmax_top")
         if T * top <= DENSE_MAX_PAIRS or _capturing(h):
-            up = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w1.transpose(1, 2)).view(E * T, Fe)
-            ys = torch.bmm(mx.relu2(up).view(E, T, Fe), self.w2.transpose(1, 2)).view(E * T, W)
+            up = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w1).view(E * T, Fe)
+            ys = torch.bmm(mx.relu2(up).view(E, T, Fe), self.w2).view(E * T, W)
             rows = torch.arange(T, dtype=torch.int32, device=h.device)[:, None]
             return mx.moe_combine(ys, (idx * T + rows).to(torch.int32), idx, wts, h, shared, E)
         flat = idx.reshape(-1).long()
@@ -408,11 +431,11 @@ class TopSoftmaxRoutedFF:
         up = torch.empty((T * top, Fe), dtype=h.dtype, device=h.device)
         live = [(e, offs[e], offs[e + 1]) for e in range(E) if offs[e + 1] > offs[e]]
         for e, a, b in live:
-            torch.mm(xs[a:b], self.w1[e].t(), out=up[a:b])
+            torch.mm(xs[a:b], self.w1[e], out=up[a:b])
         act = mx.relu2(up)                                   # one activation launch over all buckets
         ys = torch.empty((T * top, W), dtype=h.dtype, device=h.device)
         for e, a, b in live:
-            torch.mm(act[a:b], self.w2[e].t(), out=ys[a:b])
+            torch.mm(act[a:b], self.w2[e], out=ys[a:b])
         pos = torch.empty_like(order)
         pos[order] = torch.arange(order.numel(), device=order.device)
         return mx.moe_combine(ys, pos.view(T, top).to(torch.int32), idx, wts, h, shared, E)
@@ -1037,9 +1060,88 @@ class PlainLatentAttentionMixer:
         return F.linear(o, self.o)
 
 
+class ConvAttentionMixer:
+    """Softmax attention with ``kv_heads`` key/value heads (query head h reads head h // (H/G)), key size ``dim``,
+    value size ``vdim``, no biases, no rotation.  The projected q, k and v each pass a causal per-channel
+    convolution of ``conv`` taps (no bias, no activation; no entry: none), then every q and k head is divided by
+    its root mean square over ``dim`` and multiplied by one weight shared by the heads; q at position p is
+    multiplied by 1 + q_temp.coef * ln(floor((p + 1) / q_temp.every) + 1) (no entry: 1).
+    score = q . k * scale - slope_h * (i - j) with slope_h = 2^(-8 (h + 1) / H); position i sees j with
+    0 <= i - j < mask.size (no ``mask`` entry: every j <= i); the softmax denominator of head h also holds
+    exp(sink_h).  The concatenated heads are multiplied element by element by sigmoid(W_g h), then W_o.
+
+    The cache holds one row [finished k | convolved v] per token, the state slot the last taps - 1 projected inputs.
+    With ``kv_from`` = j the layer has no keys and values of its own: it attends over layer j's cache rows
+    (``forward``'s ``kv_cache``) and convolves its queries only."""
+    kind = "conv_attention"
+
+    def __init__(self, spec: Dict, width: int, eps: float):
+        self.H, self.G = int(spec["heads"]), int(spec.get("kv_heads", spec["heads"]))
+        self.D, self.P = int(spec["dim"]), int(spec["vdim"])
+        self.K = int(spec.get("conv") or 0)
+        self.taps = max(self.K, 1)
+        self.kv_from = None if spec.get("kv_from") is None else int(spec["kv_from"])
+        mask = spec.get("mask") or {}
+        self.window = int(mask["size"]) if mask.get("size") else 1 << 30
+        temp = spec.get("q_temp") or {}
+        self.temp = (float(temp.get("coef", 0.0)), int(temp.get("every", 1)))
+        self.scale = float(spec["scale"]) if "scale" in spec else self.D ** -0.5
+        self.width, self.eps = width, eps
+        if self.H % self.G or self.D > 512 or self.P > 512:
+            raise ValueError("attention: heads must split into kv_heads; dim, vdim <= 512")
+        if self.taps > 16 or self.temp[1] < 1:
+            raise ValueError("attention: at most 16 convolution taps, q_temp.every >= 1")
+        g = self.G if self.kv_from is None else 0
+        self.nq, self.nk, self.nv, self.no = self.H * self.D, g * self.D, g * self.P, self.H * self.P
+        self.C = self.nq + self.nk + self.nv                 # convolved channels: q | k | v
+        self.in_rows = self.C + self.no                      # ... | gate
+
+    def shapes(self) -> Dict[str, tuple]:
+        W = self.width
+        s = {"q": (self.nq, W), "q.norm": (self.D,), "sink": (self.H,), "g": (self.no, W), "o": (W, self.no)}
+        if self.kv_from is None:
+            s.update({"k": (self.nk, W), "k.norm": (self.D,), "v": (self.nv, W)})
+        if self.K:
+            s["q.conv"] = (self.nq, self.K)
+            if self.kv_from is None:
+                s.update({"k.conv": (self.nk, self.K), "v.conv": (self.nv, self.K)})
+        return s
+
+    def cache_spec(self):
+        rows = ("rows", self.nk + self.nv) if self.kv_from is None else ("none",)
+        return ("pair", rows, ("slots", {"conv": (self.K - 1, self.C)} if self.K > 1 else {}))
+
+    def load(self, get: Getter, dtype) -> torch.Tensor:
+        names = ("q",) if self.kv_from is not None else ("q", "k", "v")
+        self.o = get("o").to(dtype).contiguous()
+        dev = self.o.device
+        self.conv_w = (torch.cat([_f32(get, n + ".conv") for n in names], 0).contiguous() if self.K
+                       else torch.ones((self.C, 1), dtype=torch.float32, device=dev))
+        self.q_norm = _f32(get, "q.norm")
+        self.k_norm = _f32(get, "k.norm") if self.kv_from is None else None
+        self.sink = _f32(get, "sink")
+        self.slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / self.H) for h in range(self.H)], dtype=torch.float32).to(dev)
+        return torch.cat([get(n) for n in names] + [get("g")], 0).to(dtype)
+
+    def num_bytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in (self.o, self.conv_w))
+
+    def forward(self, proj: torch.Tensor, positions: torch.Tensor, meta: AttentionMetadata, cache,
+                kv_cache=None) -> torch.Tensor:
+        rows = (cache if self.kv_from is None else kv_cache)[1][1]
+        own = self.kv_from is None
+        q = mx.conv_heads(proj, self.conv_w, cache[2][1].get("conv"), self.q_norm, self.k_norm, self.eps, meta.seg_cu,
+                          meta.seg_state, positions, meta.slots, rows if own else None, meta.seg_max_len, self.H,
+                          self.G if own else 0, self.D, self.P, *self.temp)
+        o = mx.window_attend(q, rows, meta.seg_cu, positions, meta.seg_bt, self.window, self.scale, meta.seg_max_len,
+                             self.H, self.G, self.D, self.P, gate=proj[:, self.C:self.C + self.no], slopes=self.slopes,
+                             sink=self.sink)
+        return F.linear(o, self.o)
+
+
 MIXERS = {"mamba2": Mamba2Mixer, "latent_attention": LatentAttentionMixer, "channel_delta": ChannelDeltaMixer,
           "gla": GLAMixer, "window_attention": WindowAttentionMixer, "gated_lru": GatedLRUMixer,
           "parallel": ParallelMixer, "lightning": LightningMixer, "retention": RetentionMixer,
           "attention": ChunkAttentionMixer, "sigmoid_attention": SigmoidAttentionMixer, "mingru": MinGRUMixer,
           "weighted_parallel": WeightedParallelMixer, "sink_window_attention": SinkWindowAttentionMixer,
-          "plain_latent_attention": PlainLatentAttentionMixer}
+          "plain_latent_attention": PlainLatentAttentionMixer, "conv_attention": ConvAttentionMixer}

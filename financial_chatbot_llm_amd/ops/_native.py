@@ -91,7 +91,10 @@ _MIXER_SIGS = {
     "mx_group_norm": [P, c_long, c_int, P, c_long, c_int, P, c_float, P, c_long, c_int, c_int, c_int, c_int, P],
     "mx_relu2": [P, c_long, P, c_long, c_int, c_int, c_int, P],
     "mx_glu_clamp": [P, c_long, P, c_long, c_float, c_float, P, c_long, c_int, c_int, c_int, P],
-    "mx_route_biased": [P, P, c_int, c_int, P, P, c_int, P],
+    "mx_route_biased": [P, P, c_int, c_int, c_int, c_int, c_float, P, P, c_int, P],
+    "mx_dyn_tanh": [P, P, c_long, P, P, c_int, c_float, c_int, c_float, P, P, c_float, P, P, P, c_int, c_int, c_int, P],
+    "mx_conv_heads": [P, c_long, c_int, P, c_int, P, P, P, c_float, c_float, c_int, P, P, P, P, P, P, c_int, c_int, c_int,
+                      c_int, c_int, c_int, P],
     "mx_moe_combine": [P, P, P, P, P, c_long, P, c_long, c_int, c_int, c_int, P, c_int, c_int, P],
     "mx_conv_silu": [P, c_long, c_int, P, P, P, P, P, P, P, c_int, c_int, c_int, c_int, P],
     "mx_conv_act": [P, c_long, c_int, P, P, P, c_int, P, P, P, P, P, c_int, c_int, c_int, c_int, P],
@@ -104,8 +107,8 @@ _MIXER_SIGS = {
                        P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mx_lru_scan": [P, P, c_int, P, P, P, P, c_long, c_int, P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
     "mx_qk_norm_write": [P, c_long, P, c_long, P, c_long, P, P, c_float, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mx_window_attend": [P, c_long, P, P, P, P, c_int, P, c_long, c_int, c_int, c_int, P, c_float, P, c_int, c_int, c_int,
-                         c_int, c_int, c_int, c_int, c_int, P, P],
+    "mx_window_attend": [P, c_long, P, P, P, P, c_int, P, c_long, c_int, c_int, c_int, c_int, P, P, P, c_float, P, c_int,
+                         c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P],
     "mx_mingru_scan": [P, c_long, P, c_long, P, c_long, c_int, P, P, P, P, P, P, P, P, P, c_int, c_int, c_int, c_int,
                        c_int, P],
     "mx_decay_scan": [P, c_long, P, c_long, c_int, P, c_long, c_int, c_int, P, c_float, P, P, P, P, P, c_int, c_int,

@@ -12,7 +12,11 @@ with one fixed decay per head, a chunked attention mask, top-k routing with a so
 logits, and the logit scale / soft cap; and, for pre-norm decoders with gated residual updates, a sigmoid
 gate and two weighted outputs on the fused residual update, attention with kept first tokens beyond a
 sliding window and with unnormalised sigmoid weights, a minimal gated recurrent unit, values blended
-across layers at the cache write, and linearly scaled rotation frequencies.
+across layers at the cache write, and linearly scaled rotation frequencies; and, for decoders whose norms are
+elementwise (dynamic tanh) on both sides of a sublayer, one pass that norms a sublayer's output into the
+stream and the stream into the next sublayer's input, a short convolution fused with per-head norms, a query
+temperature and the cache write, distance biases, softmax sinks and elementwise output gates in the attention,
+and routing with renormalised, scaled weights.
 
 Activations are bf16 or f32 (a model-wide choice); statistics, scores, softmax, recurrences and the
 residual stream are f32 either way.  CUDA(HIP) tensors run the kernels of ``libpenny_mixers.so``
@@ -25,7 +29,7 @@ segment whose first row is at position 0 starts from zero state whatever its slo
 """
 from __future__ import annotations
 
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple
 
 import torch
 import torch.nn.functional as F
@@ -103,6 +107,56 @@ def residual_norm(x: torch.Tensor, w: Optional[torch.Tensor], eps: float, a: Opt
     return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
 
 
+class DynTanh(NamedTuple):
+    """Parameters of the elementwise norm tanh(alpha * x) * w + b (no statistics): ``w`` and ``b`` f32 [W]."""
+    alpha: float
+    w: torch.Tensor
+    b: torch.Tensor
+
+    def plain(self, v: torch.Tensor) -> torch.Tensor:
+        return torch.tanh(self.alpha * v) * self.w.float() + self.b.float()
+
+
+def _dyn_tanh_call(x, a, ids, table, scale, pre, post, out):
+    T, W = x.shape
+    src = a if a is not None else table
+    N.mcall("mx_dyn_tanh", N.ptr(x), N.ptr(_rows(a)) if a is not None else None, a.stride(0) if a is not None else 0,
+            N.ptr(ids), N.ptr(table), table.shape[0] if table is not None else 0, float(scale),
+            _dt(src) if src is not None else 1, pre.alpha if pre is not None else 0.0, N.ptr(pre.w) if pre is not None else None,
+            N.ptr(pre.b) if pre is not None else None, post.alpha if post is not None else 0.0,
+            N.ptr(post.w) if post is not None else None, N.ptr(post.b) if post is not None else None, N.ptr(out),
+            _dt(out) if out is not None else 1, T, W, N.stream())
+
+
+def dyn_tanh_embed(ids: torch.Tensor, table: torch.Tensor, scale: float, norm: DynTanh, post: Optional[DynTanh] = None,
+                   out_dtype: torch.dtype = torch.bfloat16) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """The f32 residual stream x = norm(table[id] * scale) [T, W] and, with ``post``, post(x) in ``out_dtype`` (the
+    first sublayer's input), in one pass."""
+    T, (V, W) = ids.numel(), table.shape
+    if N.use_native(table):
+        x = torch.empty((T, W), dtype=torch.float32, device=table.device)
+        out = torch.empty((T, W), dtype=out_dtype, device=table.device) if post is not None else None
+        _dyn_tanh_call(x, None, ids.to(torch.int32).contiguous(), table.contiguous(), scale, norm, post, out)
+        return x, out
+    x = norm.plain(table[ids.long().clamp(0, V - 1)].float() * scale)
+    return x, post.plain(x).to(out_dtype) if post is not None else None
+
+
+def dyn_tanh_residual(x: torch.Tensor, y: Optional[torch.Tensor], norm: Optional[DynTanh], post: Optional[DynTanh] = None,
+                      out_dtype: torch.dtype = torch.bfloat16) -> Optional[torch.Tensor]:
+    """``x`` (f32 [T, W], in place) <- x + norm(y) for a sublayer's output ``y`` (None: x stays), then post(x) in
+    ``out_dtype`` (the next sublayer's input; ``post`` None: the update only), in one pass."""
+    T, W = x.shape
+    assert x.dtype == torch.float32 and x.is_contiguous() and (y is None or (y.shape == x.shape and norm is not None))
+    if N.use_native(x):
+        out = torch.empty((T, W), dtype=out_dtype, device=x.device) if post is not None else None
+        _dyn_tanh_call(x, y, None, None, 1.0, norm if y is not None else None, post, out)
+        return out
+    if y is not None:
+        x.add_(norm.plain(y.float()))
+    return post.plain(x).to(out_dtype) if post is not None else None
+
+
 def group_norm(inp: torch.Tensor, w: torch.Tensor, eps: float, groups: int = 1, gate: Optional[torch.Tensor] = None,
                out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
     """RMS norm of each of ``groups`` equal parts of every row of ``inp`` [T, n] (each part by its own
@@ -154,22 +208,31 @@ def glu_clamp(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float) 
 # ----------------------------------------------------------------------------------------------
 # routing
 # ----------------------------------------------------------------------------------------------
-def route_biased(z: torch.Tensor, bias: Optional[torch.Tensor], top: int) -> Tuple[torch.Tensor, torch.Tensor]:
-    """Scores s = softmax(z) over all entries (f32); the ``top`` entries with the largest s + bias are
-    chosen, and their weights are the unbiased scores s (not renormalised).  Returns (weights f32
+def route_biased(z: torch.Tensor, bias: Optional[torch.Tensor], top: int, score: str = "softmax", renorm: bool = False,
+                 scale: float = 1.0) -> Tuple[torch.Tensor, torch.Tensor]:
+    """Scores s of the f32 router logits ``z``: softmax over all entries, or (``score="sigmoid"``) the sigmoid of
+    each; the ``top`` entries with the largest s + bias are chosen, and their weights are the unbiased scores s --
+    with ``renorm`` divided by the chosen scores' sum (+ 1e-20) -- times ``scale``.  Returns (weights f32
     [T, top], indices int32 [T, top])."""
     T, E = z.shape
     assert z.dtype == torch.float32
+    if score not in ("softmax", "sigmoid"):
+        raise ValueError(f"unknown routing score {score!r}")
     if N.use_native(z):
         z = z.contiguous()
         w = torch.empty((T, top), dtype=torch.float32, device=z.device)
         i = torch.empty((T, top), dtype=torch.int32, device=z.device)
-        N.mcall("mx_route_biased", N.ptr(z), N.ptr(bias), E, top, N.ptr(w), N.ptr(i), T, N.stream())
+        N.mcall("mx_route_biased", N.ptr(z), N.ptr(bias), E, top, 1 if score == "sigmoid" else 0, 1 if renorm else 0,
+                float(scale), N.ptr(w), N.ptr(i), T, N.stream())
         return w, i
-    s = torch.softmax(z, -1)
+    s = torch.sigmoid(z) if score == "sigmoid" else torch.softmax(z, -1)
     c = s + bias.float() if bias is not None else s
-    idx = torch.topk(c, top, dim=-1).indices
-    return s.gather(1, idx), idx.to(torch.int32)
+    # a stable sort: ties go to the lower index, as in the kernel
+    idx = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
+    w = s.gather(1, idx)
+    if renorm:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    return w * scale, idx.to(torch.int32)
 
 
 def moe_combine(ys: Optional[torch.Tensor], pos: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, h: torch.Tensor,
@@ -739,10 +802,67 @@ def qk_norm_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, qw: Optiona
     return rms(q, qw).to(q.dtype) if qw is not None else q
 
 
+def conv_heads(proj: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], q_norm: Optional[torch.Tensor],
+               k_norm: Optional[torch.Tensor], eps: float, cu: torch.Tensor, slot: torch.Tensor, pos: torch.Tensor,
+               slots: torch.Tensor, cache: Optional[torch.Tensor], max_len: int, heads: int, kv_heads: int, dim: int,
+               vdim: int, temp_coef: float = 0.0, temp_every: int = 1) -> torch.Tensor:
+    """Projected heads up to attention.  ``proj`` [T, C] (a column slice) holds the channels q: H*dim | k: G*dim |
+    v: G*vdim; every channel is convolved causally over its segment with ``w`` f32 [C, K] (last column: the current
+    token's tap, no activation; ``state`` f32 [slots, K-1, C]: each slot's last K-1 inputs, read unless the
+    segment starts at position 0, then replaced; unused for K = 1).  Then each q and k head is divided by its root
+    mean square over ``dim`` and multiplied by ``q_norm`` / ``k_norm`` f32 [dim] (None: neither), q by
+    1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) at position p.  The finished k and the convolved v go to
+    ``cache`` row ``slots[t]`` as [k | v] (< 0: no write); q is returned [T, H*dim].  ``kv_heads`` 0: queries
+    only, no cache row (a layer that reads another layer's keys and values)."""
+    T = proj.shape[0]
+    H, G, D, P = heads, kv_heads, dim, vdim
+    K = w.shape[1]
+    C = (H + G) * D + G * P
+    S = cu.numel() - 1
+    assert w.dtype == torch.float32 and w.shape[0] == C and proj.shape[1] >= C
+    assert K == 1 or (state is not None and tuple(state.shape[1:]) == (K - 1, C))
+    assert G == 0 or cache.shape[-1] == G * (D + P)
+    if N.use_native(proj):
+        assert G == 0 or cache.dtype == proj.dtype
+        out = torch.empty((T, H * D), dtype=proj.dtype, device=proj.device)
+        N.mcall("mx_conv_heads", N.ptr(_rows(proj)), proj.stride(0), _dt(proj), N.ptr(w), K, N.ptr(state) if K > 1 else None,
+                N.ptr(q_norm), N.ptr(k_norm), float(eps), float(temp_coef), int(temp_every), N.ptr(cu), N.ptr(slot),
+                N.ptr(pos), N.ptr(slots), N.ptr(cache) if G else None, N.ptr(out), S, int(max_len), H, G, D, P, N.stream())
+        return out
+    u = proj[:, :C].float()
+    y = torch.zeros((T, C), dtype=torch.float32)
+    cul, sll, pl = cu.tolist(), slot.tolist(), pos.tolist()
+    for s in range(S):
+        a, b = cul[s], cul[s + 1]
+        if b <= a:
+            continue
+        old = K > 1 and sll[s] >= 0 and pl[a] != 0
+        full = torch.cat([state[sll[s]] if old else torch.zeros((K - 1, C)), u[a:b]])
+        y[a:b] = (full.unfold(0, K, 1) * w.float()[None]).sum(-1)
+        if K > 1 and sll[s] >= 0:
+            state[sll[s]] = full[-(K - 1):]
+
+    def normed(t, nh, nw):
+        t = t.reshape(T, nh, D)
+        if nw is not None:
+            t = t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps) * nw.float()
+        return t.reshape(T, nh * D)
+
+    q = normed(y[:, :H * D], H, q_norm)
+    if temp_coef:
+        q = q * (1.0 + temp_coef * torch.log(((pos.long() + 1) // temp_every + 1).float()))[:, None]
+    if G:
+        rows = torch.cat([normed(y[:, H * D:(H + G) * D], G, k_norm), y[:, (H + G) * D:]], 1).to(cache.dtype)
+        ok = slots >= 0
+        cache.view(-1, G * (D + P))[slots[ok].long()] = rows[ok]
+    return q.to(proj.dtype)
+
+
 def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: torch.Tensor, bt: torch.Tensor,
                   window: int, scale: float, max_len: int, heads: int, kv_heads: int, dim: int, vdim: int,
                   gate: Optional[torch.Tensor] = None, chunked: bool = False, keep_first: int = 0,
-                  head_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  head_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None,
+                  sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention of ``q`` [T, H*dim] over the cache rows [k: G*dim | v: G*vdim] of each
     segment's pages: the query at position p sees keys j with 0 <= p - j < window, or -- ``chunked`` --
     the keys j <= p with floor(j / window) == floor(p / window) (blocks of ``window`` positions counted
@@ -750,13 +870,22 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
     visible to every later query as well (at their true positions).  Query head h
     reads key/value head h // (H/G); score = q . k * scale, f32 softmax -- or, with ``head_bias`` (f32 [H]),
     no softmax: the weight of a visible key is sigmoid(score + head_bias[h]), not normalised over the keys.
-    Head h's output is multiplied by sigmoid(gate[t, h]) when a gate [T, H] is given.  Returns [T, H*vdim]."""
+    ``slopes`` (f32 [H]): a distance bias, slopes[h] * (p - j) is taken off the scaled score.  ``sink`` (f32 [H],
+    softmax only): the denominator of head h also holds exp(sink[h]).  Head h's output is multiplied by
+    sigmoid(gate[t, h]) when a gate [T, H] is given, or element by element by sigmoid(gate) when the gate is
+    [T, H*vdim].  Returns [T, H*vdim]."""
     T = q.shape[0]
     H, G, D, P = heads, kv_heads, dim, vdim
     S = cu.numel() - 1
     Wr = G * (D + P)
-    if head_bias is not None and (head_bias.dtype != torch.float32 or head_bias.numel() != H):
-        raise ValueError("head_bias: one f32 value per query head")
+    for name, t in (("head_bias", head_bias), ("slopes", slopes), ("sink", sink)):
+        if t is not None and (t.dtype != torch.float32 or t.numel() != H):
+            raise ValueError(f"{name}: one f32 value per query head")
+    if sink is not None and head_bias is not None:
+        raise ValueError("a sink belongs to the softmax denominator; sigmoid weights have none")
+    if gate is not None and gate.shape[1] not in (H, H * P):
+        raise ValueError("gate: one value per head or per output element")
+    gate_elem = gate is not None and P > 1 and gate.shape[1] == H * P
     if N.use_native(q):
         assert bt.is_contiguous() and q.dtype == cache.dtype
         out = torch.empty((T, H * P), dtype=q.dtype, device=q.device)
@@ -770,7 +899,8 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
                 ws = torch.empty((T, H, nsplit, P + 2), dtype=torch.float32, device=q.device)
         N.mcall("mx_window_attend", N.ptr(_rows(q)), q.stride(0), N.ptr(cache), N.ptr(cu), N.ptr(pos), N.ptr(bt), bt.shape[1],
                 N.ptr(_rows(gate)) if gate is not None else None, gate.stride(0) if gate is not None else 0,
-                int(min(window, 1 << 30)), 1 if chunked else 0, int(keep_first), N.ptr(head_bias), float(scale), N.ptr(out),
+                1 if gate_elem else 0, int(min(window, 1 << 30)), 1 if chunked else 0, int(keep_first), N.ptr(head_bias),
+                N.ptr(slopes), N.ptr(sink), float(scale), N.ptr(out),
                 _dt(q), S, int(max_len), H, G, D, P, nsplit, N.ptr(ws), N.stream())
         return out
     out = torch.zeros((T, H, P), dtype=torch.float32)
@@ -789,14 +919,19 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
         sc = torch.einsum("nhd,jhd->nhj", q[a:b].float().view(-1, H, D), keys) * scale
         p = pos[a:b].long()[:, None]
         j = torch.arange(ctx)[None]
+        if slopes is not None:
+            sc = sc - slopes.float()[None, :, None] * (p - j).float()[:, None, :]
         vis = (j <= p) & (((j // window == p // window) if chunked else (j > p - window)) | (j < keep_first))
         if head_bias is not None:
             wt = torch.sigmoid(sc + head_bias.float()[None, :, None]) * vis[:, None, :]
         else:
-            wt = torch.softmax(sc.masked_fill(~vis[:, None, :], float("-inf")), -1)
+            sc = sc.masked_fill(~vis[:, None, :], float("-inf"))
+            if sink is not None:                # one more entry of the denominator, without a value
+                sc = torch.cat([sc, sink.float()[None, :, None].expand(sc.shape[0], H, 1)], -1)
+            wt = torch.softmax(sc, -1)[..., :ctx]
         out[a:b] = torch.einsum("nhj,jhp->nhp", wt, vals)
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())[:, :, None]
+        out = out * torch.sigmoid(gate.float()).view(T, H, P if gate_elem else 1)
     return out.reshape(T, H * P).to(q.dtype)
 
 
