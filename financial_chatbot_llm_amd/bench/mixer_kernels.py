@@ -1,6 +1,6 @@
 """Times the sequence-mixer kernels (``ops.mixers``) at the layer shapes of a hybrid decoder.
 
-    python -m financial_chatbot_llm_amd.bench.mixer_kernels [--width 2048] [--design gezavik|sigudra|tukedra|purozen]
+    python -m financial_chatbot_llm_amd.bench.mixer_kernels [--width 2048] [--design gezavik|sigudra|tukedra|purozen|fanotar]
 
 Two step shapes: a prefill step of two 2048-token prompts and a decode step of 64 single rows at
 depth 1024.  Shapes follow ``models.gezavik.example_config(scale_up=True)``: Mamba-2 with inner =
@@ -17,6 +17,9 @@ design's kernels at ``models.tukedra.example_config(scale_up=True)`` shapes (wid
 (width / 128 heads of 128 with 4 query heads per key/value head: sigmoid-weight attention over the whole
 prefix, softmax attention with 64 rotated entries, window 1024 and 4 kept first tokens; a minimal GRU as
 wide as the model; position-free latent attention of rank 256; the gated residual update; plain GeLU).
+``--design fanotar``: that design's kernels at ``models.fanotar.example_config(scale_up=True)`` shapes (width / 128
+heads of 128 with 4 query heads per key/value head, 4 taps, window 1024 with distance bias, sink and elementwise
+gate; the elementwise norms around a sublayer; clamped units; routing over 32 experts, top 4).
 """
 from __future__ import annotations
 
@@ -261,11 +264,69 @@ def purozen(width: int) -> int:
     return 0
 
 
+def fanotar(width: int) -> int:
+    dev = "cuda"
+    H, D, P, window, K = max(width // 128, 2), 128, 128, 1024, 4
+    G = max(H // 4, 1)
+    out = lambda **kw: print(json.dumps(kw), flush=True)  # noqa: E731
+    for name, lens, start, cu, pos, slot in _steps(dev):
+        S, T, ml = len(lens), sum(lens), max(lens)
+        pages = (start + ml + 63) // 64
+        bt = torch.arange(S * pages, dtype=torch.int32, device=dev).view(S, pages).contiguous()
+        slots = (bt[:, None, :].expand(S, ml, pages).reshape(-1, pages).gather(1, (pos // 64).long()[:, None])[:, 0] * 64
+                 + pos % 64).to(torch.int32)
+        cache = torch.randn(S * pages * 64, G * (D + P), device=dev).bfloat16()
+        C = (H + G) * D + G * P
+        proj = torch.randn(T, C + H * P, device=dev).bfloat16()
+        w, st = torch.randn(C, K, device=dev), torch.zeros(S, K - 1, C, device=dev)
+        nw = torch.ones(D, device=dev)
+        conv = lambda: mx.conv_heads(proj, w, st, nw, nw, 1e-5, cu, slot, pos, slots, cache, ml, H, G, D, P, 0.1, 1024)  # noqa: E731
+        us = _time(conv)
+        out(shape=name, kernel="conv_heads", us=round(us, 1), TB_per_s=round(T * C * 4 / us / 1e6, 2))
+        stq = torch.zeros(S, K - 1, H * D, device=dev)
+        wq = w[:H * D].contiguous()
+        us = _time(lambda: mx.conv_heads(proj, wq, stq, nw, None, 1e-5, cu, slot, pos, slots, None, ml, H, 0, D, P, 0.1, 1024))
+        out(shape=name, kernel="conv_heads queries only", us=round(us, 1), TB_per_s=round(T * H * D * 4 / us / 1e6, 2))
+        q = conv()
+        sl, sink = torch.full((H,), 0.05, device=dev), torch.zeros(H, device=dev)
+        gate = proj[:, C:]
+        pairs = sum(min(p + 1, window) for n in lens for p in range(start, start + n))
+        for label, kw in (("bias + sink + elementwise gate", dict(gate=gate, slopes=sl, sink=sink)), ("plain (same walk)", {})):
+            us = _time(lambda: mx.window_attend(q, cache, cu, pos, bt, window, D ** -0.5, ml, H, G, D, P, **kw), 5)
+            out(shape=name, kernel=f"window_attend {label}", us=round(us, 1),
+                bf16_TFLOP_per_s=round(pairs * H * 2 * (D + P) / us / 1e6, 1),
+                cache_TB_per_s=round(S * min(start + ml, window + ml) * G * (D + P) * 2 / us / 1e6, 3))
+        x = torch.randn(T, width, device=dev)
+        y = torch.randn(T, width, device=dev).bfloat16()
+        one, zero = torch.ones(width, device=dev), torch.zeros(width, device=dev)
+        n1, n2 = mx.DynTanh(0.5, one, zero), mx.DynTanh(0.7, one, zero)
+        us = _time(lambda: mx.dyn_tanh_residual(x, y, n1, n2))
+        out(shape=name, kernel="dyn_tanh_residual", us=round(us, 1), TB_per_s=round(T * width * 12 / us / 1e6, 2))
+        table = torch.randn(32768, width, device=dev).bfloat16()
+        ids = torch.randint(0, 32768, (T,), dtype=torch.int32, device=dev)
+        us = _time(lambda: mx.dyn_tanh_embed(ids, table, 2.0, n1, n2))
+        out(shape=name, kernel="dyn_tanh_embed", us=round(us, 1), TB_per_s=round(T * width * 8 / us / 1e6, 2))
+        ff = 3 * width
+        gu = torch.randn(T, 2 * ff, device=dev).bfloat16()
+        us = _time(lambda: mx.glu_clamp(gu[:, :ff], gu[:, ff:], 7.0, 1.702))
+        out(shape=name, kernel="glu_clamp", us=round(us, 1), TB_per_s=round(T * ff * 6 / us / 1e6, 2))
+        us = _time(lambda: mx.glu_act(gu[:, :ff], gu[:, ff:], "silu"))
+        out(shape=name, kernel="glu_act silu (same shape)", us=round(us, 1), TB_per_s=round(T * ff * 6 / us / 1e6, 2))
+        z, corr = torch.randn(T, 32, device=dev), torch.zeros(32, device=dev)
+        us = _time(lambda: mx.route_biased(z, corr, 4, "sigmoid", True, 2.5))
+        out(shape=name, kernel="route_biased sigmoid, renormalised", us=round(us, 1))
+        us = _time(lambda: mx.route_scores(z, 4, "softmax_top"))
+        out(shape=name, kernel="route_scores softmax_top", us=round(us, 1))
+    return 0
+
+
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--width", type=int, default=2048)
-    ap.add_argument("--design", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen"])
+    ap.add_argument("--design", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen", "fanotar"])
     a = ap.parse_args(argv)
+    if a.design == "fanotar":
+        return fanotar(a.width)
     if a.design == "purozen":
         return purozen(a.width)
     if a.design == "sigudra":

@@ -4,6 +4,7 @@
     python bench.py --model-throughput sigudra          # beside Gezavik, its closest relative here
     python bench.py --model-throughput tukedra          # beside Sigudra, its closest relative here
     python bench.py --model-throughput purozen          # beside a dense-feed-forward Sigudra of equal size
+    python bench.py --model-throughput fanotar          # beside an attention-only Tukedra of equal size
     python -m financial_chatbot_llm_amd.bench.model_throughput --mt-only gezavik-w2048
 
 For each width a Gezavik model (random weights, 8 layers: latent attention and Mamba-2 mixers, dense
@@ -112,6 +113,20 @@ def register_purozen(width: int, vocab: int = 32768) -> List[str]:
     return [name, twin]
 
 
+def register_fanotar(width: int, vocab: int = 32768) -> List[str]:
+    """Register ``fanotar-w<width>`` (8 layers ``AEkKAEkK``: convolved windowed attention, every second pair of layers
+    on the keys and values of the layer before; dense and routed clamped units) and ``tukedra-att-w<width>``, the
+    Tukedra model of the same width, depth and vocabulary with attention layers only and one residual stream
+    (``aAaAaAaA``: dense and routed feed-forwards of equal shapes); returns the two names."""
+    from ..models.configs import REGISTRY, layered_config
+    from ..models.fanotar import example_config
+    from ..models.tukedra import example_config as tukedra_config
+    name, twin = f"fanotar-w{width}", f"tukedra-att-w{width}"
+    REGISTRY[name] = layered_config(example_config(width=width, vocab=vocab, pattern="AEkKAEkK", scale_up=True), name)
+    REGISTRY[twin] = layered_config(tukedra_config(width=width, vocab=vocab, pattern="aAaAaAaA", scale_up=True, streams=0), twin)
+    return [name, twin]
+
+
 def _tokens(n: int, vocab: int, seed: int) -> List[int]:
     g = torch.Generator().manual_seed(seed)
     return torch.randint(5, vocab - 300, (n,), generator=g).tolist()
@@ -183,7 +198,8 @@ def run(a) -> int:
     names: List[str] = []
     design = getattr(a, "model_throughput", "") or "gezavik"
     for w in (int(x) for x in a.mt_widths.split(",") if x):
-        names += {"sigudra": register_sigudra, "tukedra": register_tukedra, "purozen": register_purozen}.get(design, register)(w)
+        names += {"sigudra": register_sigudra, "tukedra": register_tukedra, "purozen": register_purozen,
+                  "fanotar": register_fanotar}.get(design, register)(w)
     if a.mt_only:
         names = [n for n in names if n == a.mt_only]
     for n in names:
@@ -194,7 +210,7 @@ def run(a) -> int:
 
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--model-throughput", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen"])
+    ap.add_argument("--model-throughput", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen", "fanotar"])
     add_arguments(ap)
     return run(ap.parse_args(argv))
 
