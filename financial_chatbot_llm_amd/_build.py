@@ -39,14 +39,11 @@ MDIR = os.path.join(PKG, "csrc", "mixers")
 MIXER_LIB = os.path.join(LIBDIR, "libpenny_mixers.so")
 ARCH = os.environ.get("PENNY_OFFLOAD_ARCH", "gfx950")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
+# packed FP32 instructions stay off in every library: some of their forms have given wrong results
 HIP_FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-munsafe-fp-atomics",
-             "-Wno-unused-result", "-DNDEBUG"]
+             "-Wno-unused-result", "-DNDEBUG", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 # debug library: device bounds checks (common.h PENNY_DASSERT) on, same code otherwise
 HIP_FLAGS_DEBUG = [f for f in HIP_FLAGS if f != "-DNDEBUG"] + ["-DPENNY_KERNEL_DEBUG"]
-
-
-# packed FP32 instructions stay off in the mixer library (f32 recurrences and softmax statistics)
-MIXER_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def kernel_lib(debug: bool = False) -> str:
@@ -69,8 +66,7 @@ def _run(cmd):
 
 def build_mixers(jobs: int = 8, verbose: bool = False) -> str:
     """``csrc/mixers`` -> ``libpenny_mixers.so`` (a few seconds)."""
-    return build_kernels(jobs, verbose, src_dir=MDIR, lib=MIXER_LIB, bdir=BUILD + "_mixers",
-                         flags=HIP_FLAGS + MIXER_FLAGS)
+    return build_kernels(jobs, verbose, src_dir=MDIR, lib=MIXER_LIB, bdir=BUILD + "_mixers")
 
 
 def build_kernels(jobs: int = 8, verbose: bool = False, debug: bool = False, src_dir: str = KDIR,
