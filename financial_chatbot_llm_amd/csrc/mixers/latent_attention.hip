@@ -8,10 +8,12 @@
 // of all heads are therefore the same cache rows (one read per key serves every head).
 //
 //   mx_latent_prep    RMS norm of the latent, rotary embedding (interleaved pairs, angle = pos *
-//                     inv_freq[i] in f32) of k_rot and of every head's q_rot, cache write.
+//                     inv_freq[i] in f32, cos and sin times mscale) of k_rot and of every head's
+//                     q_rot, cache write.
 //   mx_latent_attend  windowed causal softmax attention: query at position p sees keys j with
 //                     0 <= p - j < window.  Scores, softmax and accumulation in f32.  The head's
-//                     output is multiplied by sigmoid(gate[t, h]) when a gate is given.
+//                     output is multiplied by sigmoid(gate[t, h]) when a gate is given; with a sink the
+//                     softmax denominator of head h also holds exp(sink[h]) (no key, no value).
 #include <stdlib.h>
 
 #include "mx_common.h"
@@ -20,19 +22,27 @@ namespace {
 
 constexpr int PAGE = 64;            // tokens per cache page
 
-// one block per token
+// one block per token; sine and cosine are evaluated once per pair and shared by the key and all heads' queries
 template <typename T>
 __global__ void latent_prep_kernel(const T* __restrict__ kv, long skv, const float* __restrict__ norm_w, float eps,
-                                   const float* __restrict__ inv_freq, int rot_dims, const int* __restrict__ pos,
+                                   const float* __restrict__ inv_freq, int rot_dims, float mscale,
+                                   const int* __restrict__ pos,
                                    const int* __restrict__ slots, T* __restrict__ cache, const T* __restrict__ q,
                                    long sq, int q_head_stride, int q_rot_off, T* __restrict__ q_rot, int H, int R,
                                    int Dr) {
+  extern __shared__ float trig[];                     // cos [rot_dims / 2] | sin [rot_dims / 2]
   __shared__ float scratch[16];
   const long t = blockIdx.x;
   const int slot = slots[t];
   const float p = (float)pos[t];
   const T* row = kv + t * skv;
-  const int D = R + Dr;
+  const int D = R + Dr, hr = rot_dims / 2;
+  for (int i = threadIdx.x; i < hr; i += blockDim.x) {
+    float sn, cs;
+    sincosf(p * inv_freq[i], &sn, &cs);
+    trig[i] = cs * mscale;
+    trig[hr + i] = sn * mscale;
+  }
   float ss = 0.f;
   for (int i = threadIdx.x; i < R; i += blockDim.x) {
     const float v = ldf(row + i);
@@ -45,9 +55,8 @@ __global__ void latent_prep_kernel(const T* __restrict__ kv, long skv, const flo
     for (int i = threadIdx.x; i < R; i += blockDim.x) stf(dst + i, ldf(row + i) * k * norm_w[i]);
     for (int i = threadIdx.x; i < Dr / 2; i += blockDim.x) {
       const float u = ldf(row + R + 2 * i), v = ldf(row + R + 2 * i + 1);
-      if (2 * i + 1 < rot_dims) {
-        float sn, cs;
-        sincosf(p * inv_freq[i], &sn, &cs);
+      if (i < hr) {
+        const float cs = trig[i], sn = trig[hr + i];
         stf(dst + R + 2 * i, u * cs - v * sn);
         stf(dst + R + 2 * i + 1, v * cs + u * sn);
       } else {
@@ -64,9 +73,8 @@ __global__ void latent_prep_kernel(const T* __restrict__ kv, long skv, const flo
     const T* qs = q + t * sq + (long)h * q_head_stride + q_rot_off;
     T* qd = q_rot + (t * H + h) * Dr;
     const float u = ldf(qs + 2 * i), v = ldf(qs + 2 * i + 1);
-    if (2 * i + 1 < rot_dims) {
-      float sn, cs;
-      sincosf(p * inv_freq[i], &sn, &cs);
+    if (i < hr) {
+      const float cs = trig[i], sn = trig[hr + i];
       stf(qd + 2 * i, u * cs - v * sn);
       stf(qd + 2 * i + 1, v * cs + u * sn);
     } else {
@@ -93,8 +101,8 @@ template <typename T>
 __global__ void __launch_bounds__(ATT_WAVES * 64)
 latent_attend_kernel(const T* __restrict__ q_lat, const T* __restrict__ q_rot, const T* __restrict__ cache,
                      const int* __restrict__ cu, const int* __restrict__ pos, const int* __restrict__ bt, int btw,
-                     const T* __restrict__ gate, long sgate, int window, float scale, T* __restrict__ out,
-                     int H, int R, int Dr, int QT, int HB, int KT, int ldk) {
+                     const T* __restrict__ gate, long sgate, const float* __restrict__ sink, int window, float scale,
+                     T* __restrict__ out, int H, int R, int Dr, int QT, int HB, int KT, int ldk) {
   extern __shared__ __align__(16) unsigned char smem[];
   const int D = R + Dr;
   T* ktile = reinterpret_cast<T*>(smem);                                  // [KT][ldk]
@@ -186,7 +194,7 @@ latent_attend_kernel(const T* __restrict__ q_lat, const T* __restrict__ q_rot, c
     const int tq = item / nh, hh = item - tq * nh;
     const long row = r0 + t0 + tq;
     const int h = h0 + hh;
-    float g = 1.0f / l[ii];
+    float g = mx_softmax_scale(m[ii], l[ii], sink, h);
     if (gate != nullptr) g *= mx_sigmoid(ldf(gate + row * sgate + h));
 #pragma unroll
     for (int c = 0; c < ATT_RPL; ++c) {
@@ -203,7 +211,9 @@ latent_attend_kernel(const T* __restrict__ q_lat, const T* __restrict__ q_rot, c
 //     S^T = K . Q^T      A: key rows from LDS (16-byte reads), B: the wave's queries, in registers
 //     online softmax     the statistics of query (lane % 16) live in that lane, f32
 //     O^T += V^T . P^T   A: the latent part of the tile, transposed in LDS; B: P straight from the
-//                        S^T registers (the MFMA's k slots 8g+i / 8g+4+i hold keys 4g+i / 16+4g+i)
+//                        S^T registers (the MFMA's k slots 8g+i / 8g+4+i hold keys 4g+i / 16+4g+i), as
+//                        one bf16 term, or (SPLIT) as two, hi + lo, so that the f32 softmax weights are
+//                        not cut to 8 bits
 // Feature dimensions are zero-padded to multiples of 32 (keys) / 16 (values) in LDS and registers.
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
@@ -211,13 +221,13 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 constexpr int MKT = 32;             // keys per tile
 constexpr int MLDV = MKT + 8;       // row stride of the transposed value tile
 
-template <int KSM, int NTM>         // up to 32*KSM key dims, 16*NTM value dims
+template <int KSM, int NTM, bool SPLIT>         // up to 32*KSM key dims, 16*NTM value dims
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2)))   // two blocks per CU: <= 256 registers
 latent_attend_mfma_kernel(const bf16* __restrict__ q_lat, const bf16* __restrict__ q_rot,
                           const bf16* __restrict__ cache, const int* __restrict__ cu, const int* __restrict__ pos,
-                          const int* __restrict__ bt, int btw, const bf16* __restrict__ gate, long sgate, int window,
-                          float scale, bf16* __restrict__ out, int H, int R, int Dr, int QT, int HB, int nsplit,
-                          float* __restrict__ ws) {
+                          const int* __restrict__ bt, int btw, const bf16* __restrict__ gate, long sgate,
+                          const float* __restrict__ sink, int window, float scale, bf16* __restrict__ out, int H, int R,
+                          int Dr, int QT, int HB, int nsplit, float* __restrict__ ws) {
   extern __shared__ __align__(16) unsigned char smem[];
   const int D = R + Dr;
   const int KS = (D + 31) / 32, NT = (R + 15) / 16;
@@ -360,7 +370,7 @@ latent_attend_mfma_kernel(const bf16* __restrict__ q_lat, const bf16* __restrict
     tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
     const float mn = fmaxf(m, tmax);
     const float corr = (m == -INFINITY) ? 0.f : expf(m - mn);
-    bf16x8 pb;
+    bf16x8 pb, pl;
     float psum = 0.f;
 #pragma unroll
     for (int kh = 0; kh < 2; ++kh)
@@ -368,7 +378,9 @@ latent_attend_mfma_kernel(const bf16* __restrict__ q_lat, const bf16* __restrict
       for (int i = 0; i < 4; ++i) {
         const float p = sc[kh][i] == -INFINITY ? 0.f : expf(sc[kh][i] - mn);
         psum += p;
-        pb[4 * kh + i] = (bf16)p;
+        const bf16 hi = (bf16)p;
+        pb[4 * kh + i] = hi;
+        if (SPLIT) pl[4 * kh + i] = (bf16)(p - (float)hi);
       }
     psum += __shfl_xor(psum, 16, 64);
     psum += __shfl_xor(psum, 32, 64);
@@ -387,6 +399,7 @@ latent_attend_mfma_kernel(const bf16* __restrict__ q_lat, const bf16* __restrict
         }
         o[nt] *= corr;
         o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb, o[nt], 0, 0, 0);
+        if (SPLIT) o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pl, o[nt], 0, 0, 0);
       }
     }
   }
@@ -407,7 +420,7 @@ latent_attend_mfma_kernel(const bf16* __restrict__ q_lat, const bf16* __restrict
     }
     return;
   }
-  float gsc = 1.0f / l;
+  float gsc = mx_softmax_scale(m, l, sink, h);
   if (gate != nullptr) gsc *= mx_sigmoid((float)gate[row * sgate + h]);
   bf16* dst = out + (row * H + h) * R;
 #pragma unroll
@@ -424,13 +437,13 @@ latent_attend_mfma_kernel(const bf16* __restrict__ q_lat, const bf16* __restrict
 
 // grid (rows, H): combine the nsplit parts of one (row, head)
 __global__ void latent_merge_kernel(const float* __restrict__ ws, const bf16* __restrict__ gate, long sgate,
-                                    bf16* __restrict__ out, int H, int R, int nsplit) {
+                                    const float* __restrict__ sink, bf16* __restrict__ out, int H, int R, int nsplit) {
   const long row = blockIdx.x;
   const int h = blockIdx.y;
   const float* w = ws + (row * H + h) * nsplit * (long)(R + 2);
-  float M = -INFINITY;
+  float M = sink != nullptr ? sink[h] : -INFINITY;
   for (int i = 0; i < nsplit; ++i) M = fmaxf(M, w[i * (R + 2) + R]);
-  float L = 0.f;
+  float L = sink != nullptr ? expf(sink[h] - M) : 0.f;      // the sink counts once, not once per part
   for (int i = 0; i < nsplit; ++i) {
     const float mi = w[i * (R + 2) + R];
     if (mi != -INFINITY) L += w[i * (R + 2) + R + 1] * expf(mi - M);
@@ -462,24 +475,27 @@ static bool mx_use_mfma() {
 // kv [T, R+Dr] slice (row stride skv); q [T, ...] with head h's rotated part at h*q_head_stride+q_rot_off
 // (row stride sq); q_rot out [T, H, Dr]; cache [pages*64, R+Dr]; all of storage type dt
 MX_API int mx_latent_prep(const void* kv, long skv, const float* norm_w, float eps, const float* inv_freq,
-                          int rot_dims, const int* pos, const int* slots, void* cache, const void* q, long sq,
+                          int rot_dims, float mscale, const int* pos, const int* slots, void* cache, const void* q, long sq,
                           int q_head_stride, int q_rot_off, void* q_rot, int dt, int T, int H, int R, int Dr,
                           hipStream_t st) {
   if (T <= 0) return 0;
-  MX_DISPATCH(dt, TT, latent_prep_kernel<TT><<<T, 256, 0, st>>>((const TT*)kv, skv, norm_w, eps, inv_freq, rot_dims,
-                                                                pos, slots, (TT*)cache, (const TT*)q, sq,
+  if (rot_dims < 0 || rot_dims > Dr || rot_dims > 8192) return (int)hipErrorInvalidValue;
+  const size_t lds = (size_t)(rot_dims / 2) * 2 * sizeof(float);
+  MX_DISPATCH(dt, TT, latent_prep_kernel<TT><<<T, 256, lds, st>>>((const TT*)kv, skv, norm_w, eps, inv_freq, rot_dims,
+                                                                mscale, pos, slots, (TT*)cache, (const TT*)q, sq,
                                                                 q_head_stride, q_rot_off, (TT*)q_rot, H, R, Dr));
   MX_RETURN_LAUNCH();
 }
 
 // q_lat [T, H, R], q_rot [T, H, Dr], out [T, H, R] contiguous; cu [S+1] row bounds of the segments,
-// pos [T] positions, bt [S, btw] page tables; gate [T, >=H] slice (row stride sgate) or null.
+// pos [T] positions, bt [S, btw] page tables; gate [T, >=H] slice (row stride sgate) or null; sink f32 [H] or
+// null.  exact != 0: the softmax weights enter the value product of the matrix-core form as two bf16 terms.
 // nsplit > 1 with a workspace ws (f32 [T, H, nsplit, R + 2]) and single-row segments: the key range of
 // each row is walked by nsplit blocks and merged (bf16 matrix-core form only; ignored otherwise).
 MX_API int mx_latent_attend(const void* q_lat, const void* q_rot, const void* cache, const int* cu, const int* pos,
-                            const int* bt, int btw, const void* gate, long sgate, int window, float scale,
-                            void* out, int dt, int S, int max_len, int H, int R, int Dr, int nsplit, float* ws,
-                            hipStream_t st) {
+                            const int* bt, int btw, const void* gate, long sgate, const float* sink, int exact,
+                            int window, float scale, void* out, int dt, int S, int max_len, int H, int R, int Dr,
+                            int nsplit, float* ws, hipStream_t st) {
   if (S <= 0 || max_len <= 0) return 0;
   if (R > 64 * ATT_RPL) return (int)hipErrorInvalidValue;
   const int D = R + Dr;
@@ -491,17 +507,21 @@ MX_API int mx_latent_attend(const void* q_lat, const void* q_rot, const void* ca
     const size_t lds = ((size_t)MKT * (KS * 32 + 8) + (size_t)NT * 16 * MLDV) * sizeof(bf16);
     if (max_len != 1 || ws == nullptr || nsplit < 1) nsplit = 1;
     dim3 grid(nsplit > 1 ? nsplit : (max_len + QT - 1) / QT, (H + HB - 1) / HB, S);
-    if (D <= 128 && R <= 128)
-      latent_attend_mfma_kernel<4, 8><<<grid, 256, lds, st>>>(
-          (const bf16*)q_lat, (const bf16*)q_rot, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate,
-          window, scale, (bf16*)out, H, R, Dr, QT, HB, nsplit, ws);
-    else
-      latent_attend_mfma_kernel<10, 16><<<grid, 256, lds, st>>>(
-          (const bf16*)q_lat, (const bf16*)q_rot, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate,
-          window, scale, (bf16*)out, H, R, Dr, QT, HB, nsplit, ws);
+#define LATENT_LAUNCH(KSM, NTM, SPLIT)                                                                                 \
+  latent_attend_mfma_kernel<KSM, NTM, SPLIT><<<grid, 256, lds, st>>>(                                                  \
+      (const bf16*)q_lat, (const bf16*)q_rot, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, sink,    \
+      window, scale, (bf16*)out, H, R, Dr, QT, HB, nsplit, ws)
+    if (D <= 128 && R <= 128) {
+      if (exact) LATENT_LAUNCH(4, 8, true);
+      else LATENT_LAUNCH(4, 8, false);
+    } else {
+      if (exact) LATENT_LAUNCH(10, 16, true);
+      else LATENT_LAUNCH(10, 16, false);
+    }
+#undef LATENT_LAUNCH
     if (nsplit > 1) {
       dim3 g2(S, H);           // single-row segments: row index == segment index
-      latent_merge_kernel<<<g2, R >= 128 ? 128 : 64, 0, st>>>(ws, (const bf16*)gate, sgate, (bf16*)out, H, R, nsplit);
+      latent_merge_kernel<<<g2, R >= 128 ? 128 : 64, 0, st>>>(ws, (const bf16*)gate, sgate, sink, (bf16*)out, H, R, nsplit);
     }
     MX_RETURN_LAUNCH();
   }
@@ -523,7 +543,7 @@ MX_API int mx_latent_attend(const void* q_lat, const void* q_rot, const void* ca
   if (lds > 64 * 1024) return (int)hipErrorInvalidValue;
   dim3 grid((max_len + QT - 1) / QT, (H + HB - 1) / HB, S);
   MX_DISPATCH(dt, TT, latent_attend_kernel<TT><<<grid, ATT_WAVES * 64, lds, st>>>(
-      (const TT*)q_lat, (const TT*)q_rot, (const TT*)cache, cu, pos, bt, btw, (const TT*)gate, sgate, window, scale,
-      (TT*)out, H, R, Dr, QT, HB, KT, ldk));
+      (const TT*)q_lat, (const TT*)q_rot, (const TT*)cache, cu, pos, bt, btw, (const TT*)gate, sgate, sink, window,
+      scale, (TT*)out, H, R, Dr, QT, HB, KT, ldk));
   MX_RETURN_LAUNCH();
 }

@@ -62,6 +62,15 @@ __device__ __forceinline__ float mx_silu(float x) { return x * mx_sigmoid(x); }
 // softplus without a clamp: log(1 + e^x), evaluated so that neither tail overflows
 __device__ __forceinline__ float mx_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
+// factor on the accumulated values of a softmax with running maximum m and sum l: 1 / l, or with a sink
+// exp(m) / (exp(m) l + exp(sink)) evaluated from the larger exponent down
+__device__ __forceinline__ float mx_softmax_scale(float m, float l, const float* sink, int h) {
+  if (sink == nullptr) return 1.0f / l;
+  const float sk = sink[h], M = fmaxf(m, sk);
+  const float f = expf(m - M);
+  return f / (l * f + expf(sk - M));
+}
+
 // tanh with one division and no branch.  |z| < 0.6: the fifth convergent of Lambert's continued fraction
 // z / (1 + z^2 / (3 + z^2 / (5 + ...))), relative error below 1e-8 there; beyond: (1 - e) / (1 + e), e = exp(-2|z|)
 __device__ __forceinline__ float mx_tanh(float z) {

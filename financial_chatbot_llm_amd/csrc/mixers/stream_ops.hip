@@ -4,6 +4,7 @@
 //         x <- x + mult * (a + b);  y = x / sqrt(mean(x^2) + eps) * w
 //     optionally with a weight per sublayer output and a sigmoid gate per element on the update:
 //         x <- x + sigmoid(gate + gate_bias) * (mult_a * a + mult_b * b)
+//     and with a token's embedding row added after the update, or the stream starting from it;
 //   * RMS norm of a strided row slice (latent norms), optionally in equal groups and with a SiLU
 //     gate applied first (the state-space mixer's output norm);
 //   * elementwise norms D(v) = tanh(alpha v) * w + b around a sublayer, one pass over the stream:
@@ -27,18 +28,21 @@ __global__ void embed_kernel(const int* __restrict__ ids, const T* __restrict__ 
 }
 
 // one block per row.  a / b: the two sublayer outputs of a parallel block (either may be null);
-// gate (may be null): pre-activations of a sigmoid gate on the update, gate_bias f32 [W] or null.
+// gate (may be null): pre-activations of a sigmoid gate on the update, gate_bias f32 [W] or null;
+// table (may be null): row ids[t] of [vocab, W] is added after the update or, fresh, replaces x.
 template <typename TA, typename TO>
 __global__ void residual_norm_kernel(float* __restrict__ x, const TA* __restrict__ a, long sa,
                                      const TA* __restrict__ b, long sb, float mult, float mult_b,
                                      const TA* __restrict__ gate, long sg, const float* __restrict__ gate_bias,
+                                     const int* __restrict__ ids, const TA* __restrict__ table, int vocab, int fresh,
                                      const float* __restrict__ w, float eps, TO* __restrict__ out, int W) {
   __shared__ float scratch[16];
   const long t = blockIdx.x;
   float* xr = x + t * W;
+  const TA* er = table != nullptr ? table + (long)min(max(ids[t], 0), vocab - 1) * W : nullptr;
   float ss = 0.f;
   for (int i = threadIdx.x; i < W; i += blockDim.x) {
-    float v = xr[i];
+    float v = fresh ? 0.f : xr[i];
     if (a != nullptr || b != nullptr) {
       float s;
       if (mult == mult_b) {
@@ -51,14 +55,79 @@ __global__ void residual_norm_kernel(float* __restrict__ x, const TA* __restrict
       }
       if (gate != nullptr) s *= mx_sigmoid(ldf(gate + t * sg + i) + (gate_bias != nullptr ? gate_bias[i] : 0.f));
       v = v + s;
-      xr[i] = v;
     }
+    if (er != nullptr) v += ldf(er + i);
+    if (a != nullptr || b != nullptr || er != nullptr) xr[i] = v;
     ss += v * v;
   }
   if (out == nullptr) return;
   ss = mx_block_sum(ss, scratch);
   const float r = 1.0f / sqrtf(ss / (float)W + eps);
   for (int i = threadIdx.x; i < W; i += blockDim.x) stf(out + t * W + i, xr[i] * r * w[i]);
+}
+
+// the same with four adjacent columns per access and the row in registers between its two passes: a thread owns NC
+// groups of columns; every row start and W are multiples of four elements
+template <typename TA, typename TO, int NC>
+__global__ void residual_norm_vec_kernel(float* __restrict__ x, const TA* __restrict__ a, long sa,
+                                         const TA* __restrict__ b, long sb, float mult, float mult_b,
+                                         const TA* __restrict__ gate, long sg, const float* __restrict__ gate_bias,
+                                         const int* __restrict__ ids, const TA* __restrict__ table, int vocab, int fresh,
+                                         const float* __restrict__ w, float eps, TO* __restrict__ out, int W) {
+  typedef float vf __attribute__((ext_vector_type(4)));
+  typedef TA va __attribute__((ext_vector_type(4)));
+  typedef TO vo __attribute__((ext_vector_type(4)));
+  __shared__ float scratch[16];
+  const long t = blockIdx.x;
+  float* xr = x + t * W;
+  const TA* er = table != nullptr ? table + (long)min(max(ids[t], 0), vocab - 1) * W : nullptr;
+  const bool upd = a != nullptr || b != nullptr;
+  vf v[NC];
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = (threadIdx.x + c * blockDim.x) * 4;
+    v[c] = vf{0.f, 0.f, 0.f, 0.f};
+    if (i >= W) continue;
+    if (!fresh) v[c] = *reinterpret_cast<const vf*>(xr + i);
+    if (upd) {
+      va av = va{}, bv = va{};
+      if (a != nullptr) av = *reinterpret_cast<const va*>(a + t * sa + i);
+      if (b != nullptr) bv = *reinterpret_cast<const va*>(b + t * sb + i);
+      vf s;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        s[e] = mult == mult_b ? mult * ((float)av[e] + (float)bv[e]) : mult * (float)av[e] + mult_b * (float)bv[e];
+      if (gate != nullptr) {
+        const va gv = *reinterpret_cast<const va*>(gate + t * sg + i);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) s[e] *= mx_sigmoid((float)gv[e] + (gate_bias != nullptr ? gate_bias[i + e] : 0.f));
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[c][e] += s[e];
+    }
+    if (er != nullptr) {
+      const va ev = *reinterpret_cast<const va*>(er + i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[c][e] += (float)ev[e];
+    }
+    if (upd || er != nullptr) *reinterpret_cast<vf*>(xr + i) = v[c];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += v[c][e] * v[c][e];
+  }
+  if (out == nullptr) return;
+  ss = mx_block_sum(ss, scratch);
+  const float r = 1.0f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = (threadIdx.x + c * blockDim.x) * 4;
+    if (i >= W) continue;
+    const vf wv = *reinterpret_cast<const vf*>(w + i);
+    vo o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (TO)(v[c][e] * r * wv[e]);
+    *reinterpret_cast<vo*>(out + t * W + i) = o;
+  }
 }
 
 // grid (rows, groups): RMS norm of `n` contiguous elements per group.  gate (optional): the
@@ -269,14 +338,36 @@ MX_API int mx_embed(const int* ids, const void* table, int dt, float* out, int T
 }
 
 // x [T, W] f32 (updated in place when a or b is given); out (may be null: update only) of type dt_out;
-// a, b and gate (a [T, >= W] slice, or null) of type dt_ab; mult weighs a, mult_b weighs b
+// a, b, gate (a [T, >= W] slice, or null) and table of type dt_ab; mult weighs a, mult_b weighs b; with a table
+// [vocab, W] the row of ids[t] is added after the update or, fresh != 0, x starts from it (its old values unread)
 MX_API int mx_residual_norm(float* x, const void* a, long sa, const void* b, long sb, int dt_ab, float mult,
-                            float mult_b, const void* gate, long sg, const float* gate_bias, const float* w, float eps,
-                            void* out, int dt_out, int T, int W, hipStream_t st) {
+                            float mult_b, const void* gate, long sg, const float* gate_bias, const int* ids,
+                            const void* table, int vocab, int fresh, const float* w, float eps, void* out, int dt_out,
+                            int T, int W, hipStream_t st) {
   if (T <= 0) return 0;
+  if ((table != nullptr && (ids == nullptr || vocab < 1)) || (fresh && table == nullptr) ||
+      (out != nullptr && w == nullptr))
+    return (int)hipErrorInvalidValue;
+  const size_t row = dt_ab == 1 ? 16 : 8;
+  const bool vec = W % 4 == 0 && W <= 8192 && sa % 4 == 0 && sb % 4 == 0 && sg % 4 == 0 &&
+                   ((size_t)a | (size_t)b | (size_t)gate | (size_t)table) % row == 0 && ((size_t)x | (size_t)w) % 16 == 0 &&
+                   (size_t)out % (dt_out == 1 ? 16 : 8) == 0;
+  if (vec) {
+    const int cols = W / 4, ntv = cols >= 512 ? 512 : (cols + 63) / 64 * 64;
+#define RESIDUAL_VEC(NC)                                                                                              \
+  MX_DISPATCH(dt_ab, TA, MX_DISPATCH(dt_out, TO, residual_norm_vec_kernel<TA, TO, NC><<<T, ntv, 0, st>>>(             \
+      x, (const TA*)a, sa, (const TA*)b, sb, mult, mult_b, (const TA*)gate, sg, gate_bias, ids, (const TA*)table,     \
+      vocab, fresh, w, eps, (TO*)out, W)))
+    if (cols <= ntv) RESIDUAL_VEC(1);
+    else if (cols <= 2 * ntv) RESIDUAL_VEC(2);
+    else RESIDUAL_VEC(4);
+#undef RESIDUAL_VEC
+    MX_RETURN_LAUNCH();
+  }
   const int nt = W >= 1024 ? 512 : 256;
   MX_DISPATCH(dt_ab, TA, MX_DISPATCH(dt_out, TO, residual_norm_kernel<TA, TO><<<T, nt, 0, st>>>(
-      x, (const TA*)a, sa, (const TA*)b, sb, mult, mult_b, (const TA*)gate, sg, gate_bias, w, eps, (TO*)out, W)));
+      x, (const TA*)a, sa, (const TA*)b, sb, mult, mult_b, (const TA*)gate, sg, gate_bias, ids,
+      (const TA*)table, vocab, fresh, w, eps, (TO*)out, W)));
   MX_RETURN_LAUNCH();
 }
 

@@ -12,12 +12,15 @@
 //     window's own tiles;
 //   * sigmoid weights: with a per-head bias array the weight of a visible key is
 //     sigmoid(score + head_bias[h]) and the weights are NOT normalised over the keys (no softmax).
-// Further options, each an optional argument: a distance bias (slope[h] * (p - j) is taken off the scaled
-// score), a sink (the softmax denominator of head h also holds exp(sink[h]), once, with no key and no value)
-// and a gate per output element instead of per head (out[t, h, :] *= sigmoid(gate[t, h*P + :])).
+// Further options, each an optional argument: a soft cap on the scaled score (cap * tanh(score / cap)), a
+// distance bias (slope[h] * (p - j) is taken off the score, or rel[h][min(p - j, L - 1)] of a table over
+// distances is added to it), a sink (the softmax denominator of head h also holds exp(sink[h]), once, with no
+// key and no value) and a gate per output element instead of per head
+// (out[t, h, :] *= sigmoid(gate[t, h*P + :])).
 //
 //   mx_qk_norm_write   RMS norm over the WHOLE query projection and over the whole key projection
-//                      (all heads at once, plain weights), cache write of [normed k | v].
+//                      (all heads at once, plain weights), then a rotation of part of each head, cache
+//                      write of [finished k | v].
 //   mx_window_attend   the attention, over a flat batch of segments (prompt chunks and single
 //                      decoded tokens alike).
 #include <stdlib.h>
@@ -39,13 +42,10 @@ __device__ __forceinline__ int walk_k0(int ti, int nsink, int first_tile, int KT
   return (ti < nsink ? ti : first_tile + ti - nsink) * KT;
 }
 
-// factor on the accumulated values of a softmax with running maximum m and sum l: 1 / l, or with a sink
-// exp(m) / (exp(m) l + exp(sink)) evaluated from the larger exponent down
-__device__ __forceinline__ float softmax_scale(float m, float l, const float* sink, int h) {
-  if (sink == nullptr) return 1.0f / l;
-  const float sk = sink[h], M = fmaxf(m, sk);
-  const float f = expf(m - M);
-  return f / (l * f + expf(sk - M));
+// cap * tanh(s / cap) of the score s = raw * scale, with ck = 2 log2(e) scale / cap: cap - 2 cap / (1 + e^(2 s / cap)).
+// The absolute error is a few 2^-24 of the cap; both tails end at +-cap without an overflow.
+__device__ __forceinline__ float soft_cap(float raw, float ck, float cap) {
+  return cap - 2.0f * cap * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(raw * ck));
 }
 
 // one block per token
@@ -83,6 +83,85 @@ __global__ void qk_norm_write_kernel(const T* __restrict__ q, long sq, const T* 
   for (int i = threadIdx.x; i < nv; i += blockDim.x) dst[nk + i] = vr[i];
 }
 
+// The same with a rotation: of each head of D entries the first `rot` are turned by the angle pos * freq[i] (times
+// mscale), pair i being the entries (i, i + rot/2) or, half == 0, (2i, 2i + 1).  Sine and cosine are evaluated
+// once per pair and token and shared by all heads.  V > 1: V-entry accesses (half layout; rot/2, D and every row
+// start are multiples of V).
+template <typename T, int V>
+__global__ void qk_norm_rope_write_kernel(const T* __restrict__ q, long sq, const T* __restrict__ k, long sk,
+                                          const T* __restrict__ v, long sv, const float* __restrict__ qw,
+                                          const float* __restrict__ kw, float eps, int D, int rot, int half,
+                                          const float* __restrict__ freq, float mscale, const int* __restrict__ pos,
+                                          const int* __restrict__ slots, T* __restrict__ cache, T* __restrict__ qout,
+                                          int nq, int nk, int nv) {
+  typedef T vec __attribute__((ext_vector_type(V)));
+  extern __shared__ float trig[];                     // cos [rot/2] | sin [rot/2]
+  __shared__ float scratch[16];
+  const long t = blockIdx.x;
+  const int hr = rot >> 1;
+  const float p = (float)pos[t];
+  for (int i = threadIdx.x; i < hr; i += blockDim.x) {
+    float sn, cs;
+    sincosf(p * freq[i], &sn, &cs);
+    trig[i] = cs * mscale;
+    trig[hr + i] = sn * mscale;
+  }
+  const T* qr = q + t * sq;
+  const T* kr = k + t * sk;
+  const auto sumsq = [&](const T* r, int n) {
+    float s = 0.f;
+    for (int i = threadIdx.x; i < n / V; i += blockDim.x) {
+      const vec x = *reinterpret_cast<const vec*>(r + (long)i * V);
+#pragma unroll
+      for (int e = 0; e < V; ++e) s += (float)x[e] * (float)x[e];
+    }
+    return mx_block_sum(s, scratch);                  // a barrier: the table above is complete
+  };
+  const float sq2 = sumsq(qr, qw != nullptr ? nq : 0), sk2 = sumsq(kr, kw != nullptr ? nk : 0);
+  const float cq = 1.0f / sqrtf(sq2 / (float)nq + eps), ck = 1.0f / sqrtf(sk2 / (float)nk + eps);
+  const int hv = hr / V, per = hv + (D - rot) / V;    // work items of one head: pairs of vectors, then the rest
+  const auto turn = [&](const T* src, const float* w, float c, T* dst, int n) {
+    const int items = n / D * per;
+    for (int e = threadIdx.x; e < items; e += blockDim.x) {
+      const int head = e / per, it = e - head * per;
+      const long o = (long)head * D;
+      if (it < hv) {
+        const int i0 = it * V;
+        const long a = o + (half ? i0 : 2 * i0), b = o + (half ? i0 + hr : 2 * i0 + 1);
+        const vec xa = *reinterpret_cast<const vec*>(src + a), xb = *reinterpret_cast<const vec*>(src + b);
+        vec ya, yb;
+#pragma unroll
+        for (int z = 0; z < V; ++z) {
+          float u = (float)xa[z], x2 = (float)xb[z];
+          if (w != nullptr) {
+            u = u * c * w[a + z];
+            x2 = x2 * c * w[b + z];
+          }
+          const float cs = trig[i0 + z], sn = trig[hr + i0 + z];
+          ya[z] = (T)(u * cs - x2 * sn);
+          yb[z] = (T)(x2 * cs + u * sn);
+        }
+        *reinterpret_cast<vec*>(dst + a) = ya;
+        *reinterpret_cast<vec*>(dst + b) = yb;
+      } else {
+        const long a = o + rot + (long)(it - hv) * V;
+        const vec xa = *reinterpret_cast<const vec*>(src + a);
+        vec ya;
+#pragma unroll
+        for (int z = 0; z < V; ++z) ya[z] = w != nullptr ? (T)((float)xa[z] * c * w[a + z]) : xa[z];
+        *reinterpret_cast<vec*>(dst + a) = ya;
+      }
+    }
+  };
+  turn(qr, qw, cq, qout + t * nq, nq);
+  const int slot = slots[t];
+  if (slot < 0) return;
+  T* dst = cache + (long)slot * (nk + nv);
+  turn(kr, kw, ck, dst, nk);
+  const T* vr = v + t * sv;
+  for (int i = threadIdx.x; i < nv; i += blockDim.x) dst[nk + i] = vr[i];
+}
+
 // Work layout: a block owns QT consecutive rows of one segment and HB query heads of ONE key/value
 // head; its QT*HB (row, head) items are dealt round-robin to the 4 waves (<= ITEMS per wave).  Tiles
 // of KT keys and values of that key/value head are staged in LDS once per block and shared by all
@@ -99,7 +178,8 @@ __global__ void __launch_bounds__(WA_WAVES * 64)
 window_attend_kernel(const T* __restrict__ q, long sq, const T* __restrict__ cache, const int* __restrict__ cu,
                      const int* __restrict__ pos, const int* __restrict__ bt, int btw, const T* __restrict__ gate,
                      long sgate, int gate_elem, int window, int chunked, int keep, const float* __restrict__ hbias,
-                     const float* __restrict__ slope, const float* __restrict__ sink, float scale, T* __restrict__ out,
+                     const float* __restrict__ slope, const float* __restrict__ rel, int rel_len, float cap,
+                     const float* __restrict__ sink, float scale, T* __restrict__ out,
                      int H, int G, int D, int P, int QT, int HB, int KT, int ldk, int ldv) {
   extern __shared__ __align__(16) unsigned char smem[];
   T* ktile = reinterpret_cast<T*>(smem);                                  // [KT][ldk]
@@ -176,7 +256,9 @@ window_attend_kernel(const T* __restrict__ q, long sq, const T* __restrict__ cac
         float a = 0.f;
         for (int d = 0; d < D; ++d) a += myq[d] * ldf(kr + d);
         sc = a * scale;
+        if (cap > 0.f) sc = cap * tanhf(sc / cap);
         if (slope != nullptr) sc -= slope[h] * (float)(p - j);
+        if (rel != nullptr) sc += rel[(long)h * rel_len + min(p - j, rel_len - 1)];
       }
       float corr = 1.f, pj;
       if (hbias != nullptr) {                              // independent sigmoid weights, no running statistics
@@ -211,7 +293,7 @@ window_attend_kernel(const T* __restrict__ q, long sq, const T* __restrict__ cac
     const int tq = item / nh, hh = item - tq * nh;
     const long row = r0 + t0 + tq;
     const int h = h0 + hh;
-    float gs = hbias != nullptr ? 1.0f : softmax_scale(m[ii], l[ii], sink, h);
+    float gs = hbias != nullptr ? 1.0f : mx_softmax_scale(m[ii], l[ii], sink, h);
     if (gate != nullptr && !gate_elem) gs *= mx_sigmoid(ldf(gate + row * sgate + h));
 #pragma unroll
     for (int c = 0; c < WA_CPL; ++c) {
@@ -250,6 +332,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
                           const int* __restrict__ cu, const int* __restrict__ pos, const int* __restrict__ bt, int btw,
                           const bf16* __restrict__ gate, long sgate, int gate_elem, int window, int chunked, int keep,
                           const float* __restrict__ hbias, const float* __restrict__ slope,
+                          const float* __restrict__ rel, int rel_len, int ldr, float cap,
                           const float* __restrict__ sink, float scale, bf16* __restrict__ out, int H, int G, int D,
                           int P, int QT, int HB, int nsplit, float* __restrict__ ws) {
   extern __shared__ __align__(16) unsigned char smem[];
@@ -317,6 +400,26 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
     t_begin = split * per;
     t_end = min(t_end, t_begin + per - 1);
   }
+  // Distance table in LDS (ldr > 0: columns reserved per head): head hh's row holds, in the order of the keys,
+  // the bias of every distance between this block's rows and keys -- entry x is the distance far - x -- so the
+  // eight scores of a lane read consecutive entries.  Without room for it the scores gather from memory.
+  float* rel_lds = reinterpret_cast<float*>(vt_lds + (size_t)NT * 16 * MLDV);
+  int rel_off = 0;
+  bool rel_tab = false;
+  if (rel != nullptr && t_begin <= t_end) {
+    const int kb = walk_k0(t_begin, nsink, first_tile, MKT);
+    const int span = (p_last - p_first) + (t_end - t_begin + 1) * MKT;
+    rel_tab = ldr > 0 && nsink == 0 && span <= ldr;
+    if (rel_tab) {
+      const int far = p_last - kb;
+      for (int e = threadIdx.x; e < nh * span; e += 256) {
+        const int hq = e / span, x = e - hq * span;
+        rel_lds[hq * ldr + x] = rel[(long)(h0 + hq) * rel_len + min(max(far - x, 0), rel_len - 1)];
+      }
+      rel_off = hh * ldr + far - max(pq, p_first) + 4 * g;      // + the key's position: its entry
+    }
+  }
+  const float cap_k = cap > 0.f ? 2.885390081777927f * scale / cap : 0.f;
   // staging, 16-byte path (D, P multiples of 8): a work item is a pair of keys x 8 dims of the key
   // part or of the value part -- two row loads; key pieces go to the key tile as two 16-byte stores,
   // value pieces to the transposed value tile as eight 4-byte stores (one key pair each).  The next
@@ -395,11 +498,27 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
 #pragma unroll
       for (int ks = 0; ks < KSM; ++ks)
         if (ks < KS) st[kh] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kr + 32 * ks), qf[ks], st[kh], 0, 0, 0);
+      if (cap > 0.f) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) sc[kh][i] = soft_cap(st[kh][i], cap_k, cap);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) sc[kh][i] = st[kh][i] * scale;
+      }
+      if (rel_tab) {
+        const float* rt = rel_lds + rel_off + k0 + 16 * kh;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) sc[kh][i] += rt[i];
+      } else if (rel != nullptr) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          sc[kh][i] += rel[(long)h * rel_len + min(max(pq - (k0 + 16 * kh + 4 * g + i), 0), rel_len - 1)];
+      }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int j = k0 + 16 * kh + 4 * g + i;
         const bool vis = j <= pq && (j >= pq_lo || j < keep);
-        sc[kh][i] = vis ? st[kh][i] * scale + slp * (dist0 + (float)(16 * kh + i)) : -INFINITY;
+        sc[kh][i] = vis ? sc[kh][i] + slp * (dist0 + (float)(16 * kh + i)) : -INFINITY;
         tmax = fmaxf(tmax, sc[kh][i]);
       }
     }
@@ -459,7 +578,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
     }
     return;
   }
-  float gsc = sigm ? 1.0f : softmax_scale(m, l, sink, h);
+  float gsc = sigm ? 1.0f : mx_softmax_scale(m, l, sink, h);
   if (gate != nullptr && !gate_elem) gsc *= mx_sigmoid((float)gate[row * sgate + h]);
   bf16* dst = out + (row * H + h) * P;
   const bf16* ge = gate_elem ? gate + row * sgate + (long)h * P : nullptr;
@@ -544,13 +663,36 @@ static bool wa_use_mfma() {
 }
 
 // q [T, nq], k [T, nk], v [T, nv] slices (row strides sq, sk, sv); qw [nq], kw [nk] f32 (null: no norm);
-// cache [pages*64, nk + nv]; qout [T, nq] contiguous, or null without a query norm (cache write only); all of
-// storage type dt
+// rot > 0: the first rot entries of each head of D entries are rotated (freq f32 [rot/2], pos [T]; half: pair
+// layout); cache [pages*64, nk + nv]; qout [T, nq] contiguous, or null without a query norm and a rotation (cache
+// write only); all of storage type dt
 MX_API int mx_qk_norm_write(const void* q, long sq, const void* k, long sk, const void* v, long sv, const float* qw,
-                            const float* kw, float eps, const int* slots, void* cache, void* qout, int dt, int T,
-                            int nq, int nk, int nv, hipStream_t st) {
+                            const float* kw, float eps, int D, int rot, int half, const float* freq, float mscale,
+                            const int* pos, const int* slots, void* cache, void* qout, int dt, int T, int nq, int nk,
+                            int nv, hipStream_t st) {
   if (T <= 0) return 0;
-  if (qout == nullptr && qw != nullptr) return (int)hipErrorInvalidValue;
+  if (qout == nullptr && (qw != nullptr || rot > 0)) return (int)hipErrorInvalidValue;
+  if (rot > 0) {
+    if (D < 1 || rot > D || (rot & 1) || nq % D || nk % D || freq == nullptr || pos == nullptr || rot > 8192)
+      return (int)hipErrorInvalidValue;
+    const size_t lds = (size_t)rot * sizeof(float);
+    const int V = dt == 1 ? 4 : 8;
+    const bool vec = half && (rot / 2) % V == 0 && D % V == 0 && sq % V == 0 && sk % V == 0 && (nk + nv) % V == 0 &&
+                     ((size_t)q | (size_t)k | (size_t)cache | (size_t)qout) % 16 == 0;
+#define QK_ROPE_LAUNCH(TT, VV)                                                                                      \
+  qk_norm_rope_write_kernel<TT, VV><<<T, 256, lds, st>>>((const TT*)q, sq, (const TT*)k, sk, (const TT*)v, sv, qw, kw, \
+                                                         eps, D, rot, half, freq, mscale, pos, slots, (TT*)cache,    \
+                                                         (TT*)qout, nq, nk, nv)
+    if (dt == 1) {
+      if (vec) QK_ROPE_LAUNCH(float, 4);
+      else QK_ROPE_LAUNCH(float, 1);
+    } else {
+      if (vec) QK_ROPE_LAUNCH(bf16, 8);
+      else QK_ROPE_LAUNCH(bf16, 1);
+    }
+#undef QK_ROPE_LAUNCH
+    MX_RETURN_LAUNCH();
+  }
   MX_DISPATCH(dt, TT, qk_norm_write_kernel<TT><<<T, 256, 0, st>>>((const TT*)q, sq, (const TT*)k, sk, (const TT*)v, sv, qw,
                                                                   kw, eps, slots, (TT*)cache, (TT*)qout, nq, nk, nv));
   MX_RETURN_LAUNCH();
@@ -561,17 +703,19 @@ MX_API int mx_qk_norm_write(const void* q, long sq, const void* k, long sk, cons
 // chunked != 0: `window` is the block size of the chunked mask instead of a sliding window's length.
 // keep > 0: the first `keep` keys of the sequence stay visible beyond the window.  head_bias (f32 [H], or
 // null): sigmoid weights sigmoid(score + head_bias[h]) without normalisation instead of a softmax.
-// slope (f32 [H], or null): score - slope[h] * (p - j).  sink (f32 [H], or null; softmax only): exp(sink[h]) in
+// cap > 0: the scaled score becomes cap * tanh(score / cap) before any bias.  slope (f32 [H], or null):
+// score - slope[h] * (p - j).  rel (f32 [H, rel_len], or null): score + rel[h][min(p - j, rel_len - 1)].  sink (f32 [H], or null; softmax only): exp(sink[h]) in
 // the denominator.  gate_elem != 0: the gate is a [T, >= H*P] slice, one value per output element.
 // nsplit > 1 with a workspace ws (f32 [T, H, nsplit, P + 2]) and single-row segments: the key range of
 // each row is walked by nsplit blocks and merged (bf16 matrix-core form only; ignored otherwise).
 MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int* cu, const int* pos, const int* bt,
                             int btw, const void* gate, long sgate, int gate_elem, int window, int chunked, int keep,
-                            const float* head_bias, const float* slope, const float* sink, float scale, void* out, int dt, int S, int max_len, int H, int G,
+                            const float* head_bias, const float* slope, const float* rel, int rel_len, float cap,
+                            const float* sink, float scale, void* out, int dt, int S, int max_len, int H, int G,
                             int D, int P, int nsplit, float* ws, hipStream_t st) {
   if (S <= 0 || max_len <= 0) return 0;
   if (P > 64 * WA_CPL || G < 1 || H % G || window < 1 || keep < 0 ||
-      (gate_elem && gate == nullptr) || (sink != nullptr && head_bias != nullptr))
+      (gate_elem && gate == nullptr) || (sink != nullptr && head_bias != nullptr) || (rel != nullptr && rel_len < 1))
     return (int)hipErrorInvalidValue;
   // 2: gate rows that 8-byte accesses may read (bf16)
   const int ge = !gate_elem ? 0 : (P % 4 == 0 && sgate % 4 == 0 && (size_t)gate % 8 == 0 ? 2 : 1);
@@ -581,17 +725,25 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
     const int HB = rep < 64 ? rep : 64;
     const int QT = max_len == 1 ? 1 : (64 / HB > 0 ? 64 / HB : 1);
     const int KS = (D + 31) / 32, NT = (P + 15) / 16;
-    const size_t lds = ((size_t)MKT * (KS * 32 + 8) + (size_t)NT * 16 * MLDV) * sizeof(bf16);
+    size_t lds = ((size_t)MKT * (KS * 32 + 8) + (size_t)NT * 16 * MLDV) * sizeof(bf16);
+    // distance table: every distance a block can meet, rows apart by 16 banks; only where 64 KB hold it
+    int ldr = 0;
+    if (rel != nullptr && keep == 0 && window <= 16384) {
+      const int need = window + 2 * QT + 64;
+      ldr = (need + 47) / 64 * 64 + 16;
+      if (lds + (size_t)HB * ldr * sizeof(float) <= 64 * 1024) lds += (size_t)HB * ldr * sizeof(float);
+      else ldr = 0;
+    }
     if (max_len != 1 || ws == nullptr || nsplit < 1) nsplit = 1;
     dim3 grid(nsplit > 1 ? nsplit : (max_len + QT - 1) / QT, G * ((rep + HB - 1) / HB), S);
     if (D <= 128 && P <= 128)
       window_attend_mfma_kernel<4, 8><<<grid, 256, lds, st>>>(
           (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked,
-          keep, head_bias, slope, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
+          keep, head_bias, slope, rel, rel_len, ldr, cap, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
     else
       window_attend_mfma_kernel<8, 16><<<grid, 256, lds, st>>>(
           (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked,
-          keep, head_bias, slope, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
+          keep, head_bias, slope, rel, rel_len, ldr, cap, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
     if (nsplit > 1) {
       dim3 g2(S, H);           // single-row segments: row index == segment index
       window_merge_kernel<<<g2, P >= 128 ? 128 : 64, 0, st>>>(ws, (const bf16*)gate, sgate, ge, sink, (bf16*)out, H, P,
@@ -620,6 +772,6 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
   dim3 grid((max_len + QT - 1) / QT, G * ((rep + HB - 1) / HB), S);
   MX_DISPATCH(dt, TT, window_attend_kernel<TT><<<grid, WA_WAVES * 64, lds, st>>>(
       (const TT*)q, sq, (const TT*)cache, cu, pos, bt, btw, (const TT*)gate, sgate, ge, window, chunked, keep, head_bias,
-      slope, sink, scale, (TT*)out, H, G, D, P, QT, HB, KT, ldk, ldv));
+      slope, rel, rel_len, cap, sink, scale, (TT*)out, H, G, D, P, QT, HB, KT, ldk, ldv));
   MX_RETURN_LAUNCH();
 }

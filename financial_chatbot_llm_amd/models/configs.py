@@ -15,7 +15,7 @@ from typing import Dict, Optional
 @dataclass(frozen=True)
 class ModelConfig:
     name: str
-    arch: str                       # "llama" | "mixtral" | "bert" | "gezavik" | "sigudra" | "tukedra" | "purozen" | "fanotar"
+    arch: str                       # "llama" | "mixtral" | "bert" | "gezavik" | "sigudra" | "tukedra" | "purozen" | "fanotar" | "sepitar"
     vocab_size: int
     hidden_size: int
     num_layers: int
@@ -39,6 +39,7 @@ class ModelConfig:
     layers: tuple = ()
     residual_mult: float = 1.0
     embedding: Optional[Dict] = None    # layered decoders: {"bigram": {buckets, mul_prev, mul_cur}} extra table, {"scale": s}
+    loop: Optional[Dict] = None         # layered decoders: {start, stop, times}, layers start .. stop - 1 run several times
     streams: int = 0                    # residual streams per token (hyper-connections); 0: one plain residual sum
     logit_scale: float = 1.0            # logits <- head x * logit_scale ...
     logit_softcap: float = 0.0          # ... then cap * tanh(logits / cap) (0: none)
@@ -87,6 +88,7 @@ def _register_layered() -> None:
     from .tukedra import example_config as tukedra_config
     from .purozen import example_config as purozen_config
     from .fanotar import example_config as fanotar_config
+    from .sepitar import example_config as sepitar_config
     for name, kw in (("gezavik-tiny", dict(width=192, vocab=1024, heads=3, pattern="amAm")),
                      ("gezavik-1b", dict(width=2048, vocab=32768, heads=16, pattern="aMmAmMaM" * 2, scale_up=True))):
         REGISTRY[name] = layered_config(example_config(**kw), name)
@@ -102,10 +104,13 @@ def _register_layered() -> None:
     for name, kw in (("fanotar-tiny", dict(width=160, vocab=704, pattern="AEkK")),
                      ("fanotar-1b", dict(width=2048, vocab=32768, pattern="AEAKAEkK" * 2, scale_up=True))):
         REGISTRY[name] = layered_config(fanotar_config(**kw), name)
+    for name, kw in (("sepitar-tiny", dict(width=160, vocab=736, pattern="LRC")),
+                     ("sepitar-1b", dict(width=2048, vocab=32768, pattern="LRCLLRCLLRC", scale_up=True))):
+        REGISTRY[name] = layered_config(sepitar_config(**kw), name)
 
 
 def get_model_config(name: str) -> ModelConfig:
-    if name.startswith(("gezavik-", "sigudra-", "tukedra-", "purozen-", "fanotar-")) and name not in REGISTRY:
+    if name.startswith(("gezavik-", "sigudra-", "tukedra-", "purozen-", "fanotar-", "sepitar-")) and name not in REGISTRY:
         _register_layered()
     if name in REGISTRY:
         return REGISTRY[name]
@@ -140,13 +145,13 @@ def from_hf(path: str, name: Optional[str] = None) -> ModelConfig:
         top_k_experts=c.get("num_experts_per_tok", 0), bos_token_id=c.get("bos_token_id", 1), eos_token_ids=eos)
 
 
-LAYERED_ARCHS = ("gezavik", "sigudra", "tukedra", "purozen", "fanotar")
+LAYERED_ARCHS = ("gezavik", "sigudra", "tukedra", "purozen", "fanotar", "sepitar")
 
 
 def layered_config(c: Dict, name: Optional[str] = None) -> ModelConfig:
     """A layered decoder's ``config.json`` (``architecture``, ``layers``: type / mixer / mlp per layer,
-    ``norm.eps``, ``residual_mult``, ``embedding``, ``streams``, ``logit_scale``, ``logit_softcap``, ``vocab``,
-    ``width``) -> :class:`ModelConfig`.  The
+    ``norm.eps``, ``residual_mult``, ``embedding``, ``loop``, ``streams``, ``logit_scale``, ``logit_softcap``,
+    ``vocab``, ``width``) -> :class:`ModelConfig`.  The
     flat head fields hold the first attention layer's sizes (informational; the layers carry their own)."""
     arch = str(c["architecture"]).lower()
     if arch not in LAYERED_ARCHS:
@@ -161,5 +166,5 @@ def layered_config(c: Dict, name: Optional[str] = None) -> ModelConfig:
     return ModelConfig(name or arch, arch, c["vocab"], c["width"], len(layers), heads, 1, hd, max(ffs, default=0),
                        max_position=1 << 24, norm_eps=float(c["norm"]["eps"]), bos_token_id=0, eos_token_ids=(),
                        layers=layers, residual_mult=float(c.get("residual_mult", 1.0)), embedding=c.get("embedding"),
-                       streams=int(c.get("streams") or 0), logit_scale=float(c.get("logit_scale", 1.0)),
+                       loop=c.get("loop"), streams=int(c.get("streams") or 0), logit_scale=float(c.get("logit_scale", 1.0)),
                        logit_softcap=float(c.get("logit_softcap") or 0.0))

@@ -1,6 +1,7 @@
 """Common part of the layered decoders (:mod:`.gezavik`, :mod:`.sigudra`, :mod:`.tukedra`, :mod:`.purozen`,
-:mod:`.fanotar`): a ``config.json`` lists the
-layers, each with one sequence mixer of :mod:`.mixers` and optionally one feed-forward; the residual
+:mod:`.fanotar`, :mod:`.sepitar`): a ``config.json`` lists the
+layers, each with one sequence mixer of :mod:`.mixers` and optionally one feed-forward; a span of layers may run
+several times in a row with the same weights (``loop``), each run with a cache or state of its own; the residual
 stream is f32 whatever the activation dtype; the checkpoint is the model directory itself (tensors
 ``embed``, ``l<i>.<norm>``, ``l<i>.mix.<name>``, ``l<i>.mlp.<name>``, ``final.norm``, ``head``; linear
 weights [out, in]).  A design subclasses :class:`LayeredDecoder` with its block structure: which
@@ -11,7 +12,7 @@ replicas work as for every model.
 from __future__ import annotations
 
 import math
-from typing import Callable, Dict, List, Optional
+from typing import Callable, Dict, List, NamedTuple, Optional
 
 import torch
 import torch.nn.functional as F
@@ -46,6 +47,23 @@ class Layer:
         return {}
 
 
+class LayerRun(NamedTuple):
+    layer: int
+    again: bool        # the first layer of a repeated pass
+
+
+def layer_runs(n: int, loop: Optional[Dict] = None) -> List[LayerRun]:
+    """The order in which ``n`` layers run: once each, or with ``loop`` {start, stop, times} the layers start .. stop - 1
+    ``times`` times in a row."""
+    if not loop:
+        return [LayerRun(i, False) for i in range(n)]
+    start, stop, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+    if not 0 <= start < stop <= n or times < 1:
+        raise ValueError(f"loop: 0 <= start < stop <= {n} layers and times >= 1")
+    order = list(range(start)) + list(range(start, stop)) * times + list(range(stop, n))
+    return [LayerRun(i, i == start and start < r < start + times * (stop - start)) for r, i in enumerate(order)]
+
+
 class LayeredDecoder:
     arch = ""
     mixer_types: Optional[tuple] = None
@@ -55,12 +73,17 @@ class LayeredDecoder:
     tp_rank = 0
     slot_arrays: Dict = {}       # per-slot records of the model as a whole: {name: (dtype, shape)}
     tied_head = False            # the vocabulary projection is the embedding table (no ``head`` tensor)
+    loops = False                # the design's forward follows ``runs`` (a config with a ``loop`` entry)
+    norm_offset = 0.0            # added to the layers' and the final norm's stored weights (1: stored around zero)
 
     def __init__(self, cfg: ModelConfig, device="cuda", dtype=torch.bfloat16):
         if cfg.arch != self.arch or not cfg.layers:
             raise ValueError(f"{cfg.name} is not a {self.arch} config")
         self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
         self.layers: List[Layer] = [self.make_layer(i, spec) for i, spec in enumerate(cfg.layers)]
+        if cfg.loop and not self.loops:
+            raise ValueError(f"{cfg.name}: {self.arch} models run every layer once (no loop entry)")
+        self.runs = layer_runs(len(self.layers), cfg.loop)     # layer runs in order; run r has cache entry r
         self.sequence_parallel = False
         self.capture: Optional[list] = None      # debugging: residual stream after every layer
         # head geometry the generic runner asks every decoder for (unused by the segment kernels)
@@ -144,8 +167,11 @@ class LayeredDecoder:
         open_ = [n for n, s in shapes.items() if any(d is None for d in s)]
         if open_:
             raise ValueError(f"random weights need every size in the config; open: {open_[:4]}")
-        sd = {n: self._random(n, s, seed, self.device).to(torch.bfloat16) for n, s in shapes.items()}
-        return self.load_state(sd)
+        sd = {n: self._random(n, s, seed, self.device) for n, s in shapes.items()}
+        if self.norm_offset:
+            for n in ["final.norm"] + [f"{l.prefix}.{k}" for l in self.layers for k in l.norms()]:
+                sd[n] = sd[n] - self.norm_offset
+        return self.load_state({n: t.to(torch.bfloat16) for n, t in sd.items()})
 
     def load_state(self, sd: Dict[str, torch.Tensor]) -> "LayeredDecoder":
         shapes = self.full_shapes()
@@ -160,7 +186,7 @@ class LayeredDecoder:
         get = lambda n: sd[n].to(dev)  # noqa: E731
         self.embed = get("embed").to(dt).contiguous()
         self.head = self.embed if self.tied_head else get("head").to(dt).contiguous()
-        self.final_norm = get("final.norm").float().contiguous()
+        self.final_norm = (get("final.norm").float() + self.norm_offset).contiguous()
         self.load_extra(get)
         for l in self.layers:
             self.load_layer(l, get)
@@ -180,7 +206,7 @@ class LayeredDecoder:
 
     # -- cache -------------------------------------------------------------------------------------
     def cache_specs(self):
-        return [l.mixer.cache_spec() for l in self.layers]
+        return [self.layers[r.layer].mixer.cache_spec() for r in self.runs]
 
     def kv_bytes_per_block(self) -> int:
         return HybridCache.bytes_per_block(self.cache_specs(), 4 if self.dtype == torch.float32 else 2)

@@ -6,6 +6,7 @@ normed input ``h`` and return a sublayer output, with their sizes and constants 
 * :class:`LatentAttentionMixer` -- attention whose keys and values are up-projections of one cached
   latent per token plus one shared rotated key part; runs in the latent space over a paged latent
   cache with a sliding window and a per-head sigmoid output gate.
+* :class:`SinkLatentAttentionMixer` -- the same with a sink in the softmax denominator instead of the gate.
 * :class:`ChannelDeltaMixer` -- gated delta rule with one decay per head and key channel (short
   convolutions on q, k, v; unit-norm q and k; low-rank decay and output-gate projections).
 * :class:`GLAMixer` -- gated linear attention: the same matrix state with a plain k v^T write and a
@@ -41,8 +42,13 @@ normed input ``h`` and return a sublayer output, with their sizes and constants 
   per-head RMS norms with a weight, a query temperature that grows with the position, a distance bias per head,
   a sliding window, a sink in the softmax denominator, an elementwise output gate; a layer may use an earlier
   layer's keys and values instead of its own.
+* :class:`RelBiasAttentionMixer` -- softmax attention with biased projections and no rotation; positions enter
+  through a learned bias per head and logarithmic distance bucket; a sliding window, an elementwise output gate.
+* :class:`CappedAttentionMixer` -- softmax attention with RMS norms over the whole query and key projections,
+  half-split rotation, soft-capped scores, a sink in the softmax denominator and a per-head output gate.
 * :class:`RoutedFF` -- mixture of clamped gated experts with biased top-k choice (softmax or sigmoid scores,
-  optionally renormalised and scaled weights), identity experts and an always-on shared expert.
+  optionally renormalised and scaled weights, or a softmax over the chosen biased logits), identity experts and an
+  always-on shared expert.
 * :class:`InputScaledRoutedFF` -- mixture of gated experts chosen by independent sigmoid scores, the
   score multiplying the expert's input.
 
@@ -130,27 +136,42 @@ class Mamba2Mixer:
 
 
 class LatentAttentionMixer:
+    """Latent attention: c_q = RMSnorm(W_dq h) * w, q = W_uq c_q laid out head by head as [dim | rot_dim]; W_dkv h =
+    [latent: kv_rank | key part: rot_dim], the latent RMS-normed (plain weight), the key part shared by all heads; per
+    head k = W_uk c, v = W_uv c; the rot_dim parts are rotated (pairs (2i, 2i+1), frequencies optionally scaled, see
+    :func:`..ops.mixers.rope_freqs`); score = (q . k + q_rot . k_rot) * scale; position i sees j with
+    0 <= i - j < mask.size (no ``mask`` entry: every j <= i); head h's output times sigmoid(W_g h)_h; W_o."""
     kind = "latent_attention"
+    gated = True               # output gate per head (tensor ``g``)
+    sinks = False              # exp(sink[h]) in the softmax denominator (tensor ``sink``)
+    exact_weights = False      # f32 softmax weights in the value product also in bf16
+    in_bias = None             # no bias on the stacked input projection
 
     def __init__(self, spec: Dict, width: int, eps: float):
         self.H, self.dn, self.dr, self.dv = int(spec["heads"]), int(spec["dim"]), int(spec["rot_dim"]), int(spec["vdim"])
         self.R, self.q_rank = int(spec["kv_rank"]), int(spec["q_rank"])
         rot = spec.get("rot") or {}
-        self.rot_dims = int(rot.get("dims", self.dr))
-        self.rot_base = float(rot.get("base", 10000.0))
+        self.rot = _Rotary({"dims": self.dr, "base": 10000.0, **rot} if self.dr else None, self.dr)
+        self.rot_dims = self.rot.dims
         mask = spec.get("mask") or {}
         self.window = int(mask["size"]) if mask.get("size") else 1 << 30      # no mask entry: plain causal
         self.scale = float(spec["scale"]) if "scale" in spec else (self.dn + self.dr) ** -0.5
-        self.in_rows = self.q_rank + self.R + self.dr + self.H                # c_q | c, k_rot | gate
+        self.in_rows = self.q_rank + self.R + self.dr + (self.H if self.gated else 0)     # c_q | c, k_rot | gate
         self.width, self.eps = width, eps
-        if self.rot_dims > self.dr or self.rot_dims % 2 or self.R > 512:
-            raise ValueError("latent_attention: rot.dims must be even and <= rot_dim, kv_rank <= 512")
+        self.sink = None
+        if self.R > 512:
+            raise ValueError("latent_attention: kv_rank <= 512")
 
     def shapes(self) -> Dict[str, tuple]:
         H, dq = self.H, self.dn + self.dr
-        return {"dq": (self.q_rank, self.width), "dq.norm": (self.q_rank,), "uq": (H * dq, self.q_rank),
-                "dkv": (self.R + self.dr, self.width), "dkv.norm": (self.R,), "uk": (H * self.dn, self.R),
-                "uv": (H * self.dv, self.R), "g": (H, self.width), "o": (self.width, H * self.dv)}
+        s = {"dq": (self.q_rank, self.width), "dq.norm": (self.q_rank,), "uq": (H * dq, self.q_rank),
+             "dkv": (self.R + self.dr, self.width), "dkv.norm": (self.R,), "uk": (H * self.dn, self.R),
+             "uv": (H * self.dv, self.R), "o": (self.width, H * self.dv)}
+        if self.gated:
+            s["g"] = (H, self.width)
+        if self.sinks:
+            s["sink"] = (H,)
+        return s
 
     def cache_spec(self):
         return ("latent", self.R + self.dr)
@@ -162,8 +183,11 @@ class LatentAttentionMixer:
         self.uk = get("uk").to(dtype).view(self.H, self.dn, self.R).contiguous()      # [H, dn, R]
         self.uv_t = get("uv").to(dtype).view(self.H, self.dv, self.R).transpose(1, 2).contiguous()  # [H, R, dv]
         self.o = get("o").to(dtype).contiguous()
-        self.inv_freq = mx.rope_inv_freq(self.rot_dims, self.rot_base, device=self.uq.device)
-        return torch.cat([get("dq"), get("dkv"), get("g")], 0).to(dtype)
+        self.rot.to(self.uq.device)
+        if self.rot.freq is None:
+            self.rot.freq = torch.zeros(0, dtype=torch.float32, device=self.uq.device)
+        self.sink = _f32(get, "sink") if self.sinks else None
+        return torch.cat([get("dq"), get("dkv")] + ([get("g")] if self.gated else []), 0).to(dtype)
 
     def num_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in (self.uq, self.uk, self.uv_t, self.o))
@@ -175,18 +199,25 @@ class LatentAttentionMixer:
         a = self.q_rank
         cq = mx.group_norm(proj[:, :a], self.dq_norm, self.eps, 1)
         kv = proj[:, a:a + R + dr]
-        gate = proj[:, a + R + dr:a + R + dr + H]
+        gate = proj[:, a + R + dr:a + R + dr + H] if self.gated else None
         q = F.linear(cq, self.uq)                                            # [T, H * (dn + dr)]
         # latent row + shared rotated key into the cache; every head's rotated query part
-        q_rot = mx.latent_prep(kv, self.dkv_norm, self.eps, self.inv_freq, self.rot_dims, positions, meta.slots, rows,
-                               q, H, dn + dr, dn, R, dr)
+        q_rot = mx.latent_prep(kv, self.dkv_norm, self.eps, self.rot.freq, self.rot_dims, positions, meta.slots, rows,
+                               q, H, dn + dr, dn, R, dr, self.rot.mscale)
         # fold each head's key up-projection into its query: q_lat[h] = W_uk[h]^T q_nope[h]
         q_nope = q.view(T, H, dn + dr)[:, :, :dn]
         q_lat = torch.bmm(q_nope.transpose(0, 1), self.uk).transpose(0, 1).contiguous()   # [T, H, R]
         o_lat = mx.latent_attend(q_lat, q_rot, rows, meta.seg_cu, positions, meta.seg_bt, self.window, self.scale,
-                                 meta.seg_max_len, gate=gate)
+                                 meta.seg_max_len, gate=gate, sink=self.sink, exact_weights=self.exact_weights)
         o = torch.bmm(o_lat.transpose(0, 1), self.uv_t).transpose(0, 1).reshape(T, H * self.dv)
         return F.linear(o, self.o)
+
+
+class SinkLatentAttentionMixer(LatentAttentionMixer):
+    """Latent attention without an output gate whose softmax denominator of head h also holds exp(sink[h]) (no key, no
+    value, not scaled); the softmax weights stay f32 in the value product."""
+    kind = "sink_latent_attention"
+    gated, sinks, exact_weights = False, True, True
 
 
 class DenseFF:
@@ -232,7 +263,9 @@ class RoutedFF:
     Router logits z = W_r h in f32; scores s = softmax(z) over the experts and the ``identity``
     experts that follow them, or (``score="sigmoid"``) each expert's own sigmoid(z); the ``top`` largest
     s + correction are chosen and weighted by s itself -- with ``renorm`` divided by the chosen scores' sum --
-    times the router's ``scale`` (default 1).  An identity expert returns its input.  Expert: g = min(W_g h, limit), u = clamp(W_u h, +-limit),
+    times the router's ``scale`` (default 1).  With ``score="softmax_top"`` the logits carry a bias (``router.b``
+    instead of ``correction``), the ``top`` largest are chosen and the weights are the softmax over the chosen
+    logits.  An identity expert returns its input.  Expert: g = min(W_g h, limit), u = clamp(W_u h, +-limit),
     W_d (g * sigmoid(alpha g) * (u + 1)).  A shared expert of the same form runs for every token."""
 
     def __init__(self, spec: Dict, width: int, alpha: float = 1.702, score: str = "softmax", renorm: bool = False):
@@ -248,9 +281,10 @@ class RoutedFF:
         self.in_rows = 2 * self.Fs                                            # shared gate | up
         if not 1 <= self.top <= self.E + self.I:
             raise ValueError("routed feed-forward: 1 <= top <= experts")
+        self.bias_name = "router.b" if score == "softmax_top" else "correction"
 
     def shapes(self) -> Dict[str, tuple]:
-        s = {"router": (self.E + self.I, self.width), "correction": (self.E + self.I,)}
+        s = {"router": (self.E + self.I, self.width), self.bias_name: (self.E + self.I,)}
         for e in range(self.E):
             s.update({f"e{e}.gate": (self.F, self.width), f"e{e}.up": (self.F, self.width),
                       f"e{e}.down": (self.width, self.F)})
@@ -261,7 +295,7 @@ class RoutedFF:
 
     def load(self, get: Getter, dtype) -> Optional[torch.Tensor]:
         self.router = get("router").float().contiguous()
-        self.correction = get("correction").float().contiguous()
+        self.correction = get(self.bias_name).float().contiguous()
         self.w13 = _expert_stack([torch.cat([get(f"e{e}.gate"), get(f"e{e}.up")], 0) for e in range(self.E)], dtype)
         self.w2 = _expert_stack([get(f"e{e}.down") for e in range(self.E)], dtype)
         if not self.Fs:
@@ -280,8 +314,11 @@ class RoutedFF:
         if self.Fs:
             shared = F.linear(mx.glu_clamp(proj[:, :self.Fs], proj[:, self.Fs:2 * self.Fs], self.limit_s, self.alpha),
                               self.down_s)
-        wts, idx = mx.route_biased(F.linear(h.float(), self.router), self.correction, top, self.score, self.renorm,
-                                   self.w_scale)
+        if self.score == "softmax_top":
+            wts, idx = mx.route_scores(F.linear(h.float(), self.router, self.correction), top, "softmax_top")
+        else:
+            wts, idx = mx.route_biased(F.linear(h.float(), self.router), self.correction, top, self.score, self.renorm,
+                                       self.w_scale)
         if T * top <= DENSE_MAX_PAIRS or _capturing(h):
             gu = torch.bmm(h.unsqueeze(0).expand(E, T, W), self.w13).view(E * T, 2 * Fe)
             act = mx.glu_clamp(gu[:, :Fe], gu[:, Fe:], self.limit, self.alpha)
@@ -1139,9 +1176,110 @@ class ConvAttentionMixer:
         return F.linear(o, self.o)
 
 
+class _GroupedAttention:
+    """Common part of softmax attention with ``kv_heads`` key/value heads (query head h reads head h // (H/G)), key
+    size ``dim``, value size ``vdim`` and a paged cache of one row [finished k | v] per token: sizes, mask
+    ({size}: a sliding window, position i sees j with 0 <= i - j < size; no entry: every j <= i) and ``scale``."""
+
+    def __init__(self, spec: Dict, width: int, eps: float):
+        self.H, self.G = int(spec["heads"]), int(spec.get("kv_heads", spec["heads"]))
+        self.D, self.P = int(spec["dim"]), int(spec["vdim"])
+        mask = spec.get("mask") or {}
+        self.window = int(mask["size"]) if mask.get("size") else 1 << 30
+        self.scale = float(spec["scale"]) if "scale" in spec else self.D ** -0.5
+        self.width, self.eps = width, eps
+        if self.H % self.G or self.D > 512 or self.P > 512:
+            raise ValueError("attention: heads must split into kv_heads; dim, vdim <= 512")
+        self.nq, self.nk, self.nv, self.no = self.H * self.D, self.G * self.D, self.G * self.P, self.H * self.P
+
+    def cache_spec(self):
+        return ("rows", self.nk + self.nv)
+
+    def num_bytes(self) -> int:
+        return self.o.numel() * self.o.element_size()
+
+
+class RelBiasAttentionMixer(_GroupedAttention):
+    """Softmax attention whose positions enter only through a learned distance bias: q = W_q h + b_q, k = W_k h + b_k,
+    v = W_v h + b_v, no rotation; score = q . k * scale + rel[bucket(i - j), head] with ``rel`` [buckets, heads] and
+    the buckets of :func:`..ops.mixers.distance_buckets` (``bias_max``: the distance from which all share the last
+    row); a sliding window; the concatenated heads are multiplied element by element by sigmoid(W_g h);
+    W_o and its bias."""
+    kind = "rel_bias_attention"
+
+    def __init__(self, spec: Dict, width: int, eps: float):
+        super().__init__(spec, width, eps)
+        self.far = float(spec["bias_max"])
+        self.in_rows = self.nq + self.nk + self.nv + self.no
+
+    def shapes(self) -> Dict[str, tuple]:
+        W = self.width
+        return {"q": (self.nq, W), "q.b": (self.nq,), "k": (self.nk, W), "k.b": (self.nk,), "v": (self.nv, W),
+                "v.b": (self.nv,), "rel": (None, self.H), "g": (self.no, W), "o": (W, self.no), "o.b": (W,)}
+
+    def load(self, get: Getter, dtype) -> torch.Tensor:
+        self.o, self.o_b = get("o").to(dtype).contiguous(), get("o.b").to(dtype).contiguous()
+        rel = get("rel").float()
+        rows = mx.distance_buckets(rel.shape[0], self.far)[:self.window].to(rel.device)
+        self.rel = rel[rows].t().contiguous()                # f32 [heads, distances]
+        self.in_bias = torch.cat([get("q.b"), get("k.b"), get("v.b"), torch.zeros_like(get("g")[:, 0])], 0).to(dtype)
+        return torch.cat([get("q"), get("k"), get("v"), get("g")], 0).to(dtype)
+
+    def forward(self, proj: torch.Tensor, positions: torch.Tensor, meta: AttentionMetadata, cache) -> torch.Tensor:
+        rows = cache[1]
+        nq, nk, nv = self.nq, self.nk, self.nv
+        q = mx.qk_norm_write(proj[:, :nq], proj[:, nq:nq + nk], proj[:, nq + nk:nq + nk + nv], None, None, self.eps,
+                             meta.slots, rows)
+        gate = proj[:, nq + nk + nv:nq + nk + nv + self.no]
+        o = mx.window_attend(q, rows, meta.seg_cu, positions, meta.seg_bt, self.window, self.scale, meta.seg_max_len,
+                             self.H, self.G, self.D, self.P, gate=gate, rel=self.rel)
+        return F.linear(o, self.o, self.o_b)
+
+
+class CappedAttentionMixer(_GroupedAttention):
+    """Softmax attention without projection biases: RMS norm over the WHOLE query and key projections (plain weights,
+    before the split into heads), then rotation of the first rot.dims entries of each head (entry i with entry
+    i + dims/2; frequencies optionally scaled, see :func:`..ops.mixers.rope_freqs`; no ``rot`` entry: none);
+    score = softcap * tanh(q . k * scale / softcap) (no entry: uncapped); every j <= i is visible unless a ``mask``
+    narrows it; the softmax denominator of head h also holds exp(sink[h]) (neither scaled nor capped); head h's
+    output times sigmoid(W_g h)_h; W_o."""
+    kind = "capped_attention"
+    in_bias = None
+
+    def __init__(self, spec: Dict, width: int, eps: float):
+        super().__init__(spec, width, eps)
+        self.rot = _Rotary(spec.get("rot"), self.D)
+        self.softcap = float(spec.get("softcap") or 0.0)
+        self.in_rows = self.nq + self.nk + self.nv + self.H
+
+    def shapes(self) -> Dict[str, tuple]:
+        W = self.width
+        return {"q": (self.nq, W), "k": (self.nk, W), "v": (self.nv, W), "q.norm": (self.nq,), "k.norm": (self.nk,),
+                "sink": (self.H,), "g": (self.H, W), "o": (W, self.no)}
+
+    def load(self, get: Getter, dtype) -> torch.Tensor:
+        self.q_norm, self.k_norm, self.sink = _f32(get, "q.norm"), _f32(get, "k.norm"), _f32(get, "sink")
+        self.o = get("o").to(dtype).contiguous()
+        self.rot.to(self.o.device)
+        return torch.cat([get("q"), get("k"), get("v"), get("g")], 0).to(dtype)
+
+    def forward(self, proj: torch.Tensor, positions: torch.Tensor, meta: AttentionMetadata, cache) -> torch.Tensor:
+        rows = cache[1]
+        nq, nk, nv = self.nq, self.nk, self.nv
+        q = mx.qk_norm_write(proj[:, :nq], proj[:, nq:nq + nk], proj[:, nq + nk:nq + nk + nv], self.q_norm, self.k_norm,
+                             self.eps, meta.slots, rows, dim=self.D, freq=self.rot.freq, pos=positions,
+                             mscale=self.rot.mscale)
+        gate = proj[:, nq + nk + nv:nq + nk + nv + self.H]
+        o = mx.window_attend(q, rows, meta.seg_cu, positions, meta.seg_bt, self.window, self.scale, meta.seg_max_len,
+                             self.H, self.G, self.D, self.P, gate=gate, sink=self.sink, softcap=self.softcap)
+        return F.linear(o, self.o)
+
+
 MIXERS = {"mamba2": Mamba2Mixer, "latent_attention": LatentAttentionMixer, "channel_delta": ChannelDeltaMixer,
           "gla": GLAMixer, "window_attention": WindowAttentionMixer, "gated_lru": GatedLRUMixer,
           "parallel": ParallelMixer, "lightning": LightningMixer, "retention": RetentionMixer,
           "attention": ChunkAttentionMixer, "sigmoid_attention": SigmoidAttentionMixer, "mingru": MinGRUMixer,
           "weighted_parallel": WeightedParallelMixer, "sink_window_attention": SinkWindowAttentionMixer,
-          "plain_latent_attention": PlainLatentAttentionMixer, "conv_attention": ConvAttentionMixer}
+          "plain_latent_attention": PlainLatentAttentionMixer, "conv_attention": ConvAttentionMixer,
+          "sink_latent_attention": SinkLatentAttentionMixer, "rel_bias_attention": RelBiasAttentionMixer,
+          "capped_attention": CappedAttentionMixer}

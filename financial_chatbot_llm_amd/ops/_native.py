@@ -86,8 +86,8 @@ c_double = ctypes.c_double
 # its own -- a model that runs only these builds and loads only these
 _MIXER_SIGS = {
     "mx_embed": [P, P, c_int, P, c_int, c_int, c_int, P],
-    "mx_residual_norm": [P, P, c_long, P, c_long, c_int, c_float, c_float, P, c_long, P, P, c_float, P, c_int, c_int,
-                         c_int, P],
+    "mx_residual_norm": [P, P, c_long, P, c_long, c_int, c_float, c_float, P, c_long, P, P, P, c_int, c_int, P, c_float, P,
+                         c_int, c_int, c_int, P],
     "mx_group_norm": [P, c_long, c_int, P, c_long, c_int, P, c_float, P, c_long, c_int, c_int, c_int, c_int, P],
     "mx_relu2": [P, c_long, P, c_long, c_int, c_int, c_int, P],
     "mx_glu_clamp": [P, c_long, P, c_long, c_float, c_float, P, c_long, c_int, c_int, c_int, P],
@@ -106,9 +106,10 @@ _MIXER_SIGS = {
     "mx_matrix_scan": [P, c_long, P, c_long, P, c_long, c_int, P, c_long, P, P, P, c_long, c_int, c_float, c_int, P, P, P, P,
                        P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mx_lru_scan": [P, P, c_int, P, P, P, P, c_long, c_int, P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mx_qk_norm_write": [P, c_long, P, c_long, P, c_long, P, P, c_float, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mx_window_attend": [P, c_long, P, P, P, P, c_int, P, c_long, c_int, c_int, c_int, c_int, P, P, P, c_float, P, c_int,
-                         c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P],
+    "mx_qk_norm_write": [P, c_long, P, c_long, P, c_long, P, P, c_float, c_int, c_int, c_int, P, c_float, P, P, P, P, c_int,
+                         c_int, c_int, c_int, c_int, P],
+    "mx_window_attend": [P, c_long, P, P, P, P, c_int, P, c_long, c_int, c_int, c_int, c_int, P, P, P, c_int, c_float, P,
+                         c_float, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P],
     "mx_mingru_scan": [P, c_long, P, c_long, P, c_long, c_int, P, P, P, P, P, P, P, P, P, c_int, c_int, c_int, c_int,
                        c_int, P],
     "mx_decay_scan": [P, c_long, P, c_long, c_int, P, c_long, c_int, c_int, P, c_float, P, P, P, P, P, c_int, c_int,
@@ -119,9 +120,9 @@ _MIXER_SIGS = {
                       c_float, c_float, P, c_int, P, c_long, c_int, P, P, c_long, c_int, P, c_long, c_float, c_int, P],
     "mx_logit_cap": [P, c_int, c_float, c_float, c_long, P],
     "mx_ssm_scan": [P, c_int, P, c_long, c_int, P, P, P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, P],
-    "mx_latent_prep": [P, c_long, P, c_float, P, c_int, P, P, P, P, c_long, c_int, c_int, P, c_int, c_int, c_int,
+    "mx_latent_prep": [P, c_long, P, c_float, P, c_int, c_float, P, P, P, P, c_long, c_int, c_int, P, c_int, c_int, c_int,
                        c_int, c_int, P],
-    "mx_latent_attend": [P, P, P, P, P, P, c_int, P, c_long, c_int, c_float, P, c_int, c_int, c_int, c_int, c_int,
+    "mx_latent_attend": [P, P, P, P, P, P, c_int, P, c_long, P, c_int, c_int, c_float, P, c_int, c_int, c_int, c_int, c_int,
                          c_int, c_int, P, P],
 }
 _MIXER_LIB: Optional[ctypes.CDLL] = None

@@ -16,7 +16,10 @@ across layers at the cache write, and linearly scaled rotation frequencies; and,
 elementwise (dynamic tanh) on both sides of a sublayer, one pass that norms a sublayer's output into the
 stream and the stream into the next sublayer's input, a short convolution fused with per-head norms, a query
 temperature and the cache write, distance biases, softmax sinks and elementwise output gates in the attention,
-and routing with renormalised, scaled weights.
+and routing with renormalised, scaled weights; and, for decoders that run a span of layers several times, the
+embedding output added again inside the residual update, a distance bias read from a table of logarithmic buckets,
+soft-capped attention scores, whole-projection norms fused with a rotation, sinks in latent attention, and
+frequencies scaled by their wavelength.
 
 Activations are bf16 or f32 (a model-wide choice); statistics, scores, softmax, recurrences and the
 residual stream are f32 either way.  CUDA(HIP) tensors run the kernels of ``libpenny_mixers.so``
@@ -71,28 +74,49 @@ def embed_f32(ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
 def residual_norm(x: torch.Tensor, w: Optional[torch.Tensor], eps: float, a: Optional[torch.Tensor] = None,
                   b: Optional[torch.Tensor] = None, mult: float = 1.0,
                   out_dtype: torch.dtype = torch.bfloat16, mult_b: Optional[float] = None,
-                  gate: Optional[torch.Tensor] = None, gate_bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                  gate: Optional[torch.Tensor] = None, gate_bias: Optional[torch.Tensor] = None,
+                  ids: Optional[torch.Tensor] = None, table: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """``x`` (f32 [T, W], in place) <- x + mult * (a + b) when a sublayer output is given, then
     y = x / sqrt(mean(x^2) + eps) * w in ``out_dtype`` (``w`` None: the update only).  ``mult_b``: b's own
     weight, the update is mult * a + mult_b * b.  ``gate`` ([T, W] column slice, the type of a) and
-    ``gate_bias`` (f32 [W]): the update is multiplied element by element by sigmoid(gate + gate_bias)."""
+    ``gate_bias`` (f32 [W]): the update is multiplied element by element by sigmoid(gate + gate_bias).
+    ``ids`` (int32 [T]) with ``table`` ([vocab, W], the type of a): the row ``table[ids]`` is added after the update."""
+    return _residual_norm(x, w, eps, a, b, mult, out_dtype, mult_b, gate, gate_bias, ids, table, False)
+
+
+def embed_norm(ids: torch.Tensor, table: torch.Tensor, w: torch.Tensor, eps: float,
+               out_dtype: torch.dtype = torch.bfloat16) -> Tuple[torch.Tensor, torch.Tensor]:
+    """Token rows of ``table`` as an f32 residual stream x [T, W] and its RMS norm in ``out_dtype``, in one pass."""
+    x = torch.empty((ids.numel(), table.shape[1]), dtype=torch.float32, device=table.device)
+    h = _residual_norm(x, w, eps, None, None, 1.0, out_dtype, None, None, None, ids, table, True)
+    return x, h
+
+
+def _residual_norm(x, w, eps, a, b, mult, out_dtype, mult_b, gate, gate_bias, ids, table, fresh):
     T, W = x.shape
     assert x.dtype == torch.float32 and x.is_contiguous()
     ab = a if a is not None else b
     mult_b = mult if mult_b is None else mult_b
     if gate is not None and ab is None:
         raise ValueError("a gate needs a sublayer output to act on")
+    if table is not None and (ids is None or ids.numel() != T or table.shape[1] != W):
+        raise ValueError("table: one id per row and rows of the stream's width")
     if N.use_native(x):
         out = torch.empty((T, W), dtype=out_dtype, device=x.device) if w is not None else None
         if a is not None and b is not None:
             assert a.dtype == b.dtype
         if gate is not None:
             assert gate.dtype == ab.dtype and gate.shape[1] == W
+        if table is not None:
+            assert table.is_contiguous() and (ab is None or table.dtype == ab.dtype)
+            ids = ids.to(torch.int32).contiguous()
+        src = ab if ab is not None else table
         N.mcall("mx_residual_norm", N.ptr(x), N.ptr(_rows(a)) if a is not None else None,
                 a.stride(0) if a is not None else 0, N.ptr(_rows(b)) if b is not None else None,
-                b.stride(0) if b is not None else 0, _dt(ab) if ab is not None else 1, float(mult), float(mult_b),
+                b.stride(0) if b is not None else 0, _dt(src) if src is not None else 1, float(mult), float(mult_b),
                 N.ptr(_rows(gate)) if gate is not None else None, gate.stride(0) if gate is not None else 0,
-                N.ptr(gate_bias), N.ptr(w), float(eps), N.ptr(out), _dt(out) if out is not None else 1, T, W, N.stream())
+                N.ptr(gate_bias), N.ptr(ids) if table is not None else None, N.ptr(table),
+                table.shape[0] if table is not None else 0, 1 if fresh else 0, N.ptr(w), float(eps), N.ptr(out), _dt(out) if out is not None else 1, T, W, N.stream())
         return out
     if ab is not None:
         s = torch.zeros_like(x)
@@ -102,6 +126,12 @@ def residual_norm(x: torch.Tensor, w: Optional[torch.Tensor], eps: float, a: Opt
         if gate is not None:
             s = s * torch.sigmoid(gate.float() + (gate_bias.float() if gate_bias is not None else 0.0))
         x.add_(s)
+    if table is not None:
+        row = table[ids.long().clamp(0, table.shape[0] - 1)].float()
+        if fresh:
+            x.copy_(row)
+        else:
+            x.add_(row)
     if w is None:
         return None
     return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
@@ -342,12 +372,12 @@ def rope_inv_freq(dims: int, base: float, device=None) -> torch.Tensor:
     return (1.0 / (base ** (i / dims))).contiguous()
 
 
-def _rotate(v: torch.Tensor, ang: torch.Tensor, dims: int) -> torch.Tensor:
+def _rotate(v: torch.Tensor, ang: torch.Tensor, dims: int, m: float = 1.0) -> torch.Tensor:
     """Interleaved-pair rotation of the first ``dims`` entries of the last axis; ``ang`` broadcasts
     against v[..., 0:dims:2]."""
     out = v.clone()
     a, b = v[..., 0:dims:2], v[..., 1:dims:2]
-    c, s = torch.cos(ang), torch.sin(ang)
+    c, s = torch.cos(ang) * m, torch.sin(ang) * m
     out[..., 0:dims:2] = a * c - b * s
     out[..., 1:dims:2] = b * c + a * s
     return out
@@ -355,42 +385,55 @@ def _rotate(v: torch.Tensor, ang: torch.Tensor, dims: int) -> torch.Tensor:
 
 def latent_prep(kv: torch.Tensor, norm_w: torch.Tensor, eps: float, inv_freq: torch.Tensor, rot_dims: int,
                 pos: torch.Tensor, slots: torch.Tensor, cache: torch.Tensor, q: torch.Tensor, heads: int,
-                head_stride: int, rot_off: int, rank: int, rot_dim: int) -> torch.Tensor:
+                head_stride: int, rot_off: int, rank: int, rot_dim: int, mscale: float = 1.0) -> torch.Tensor:
     """Per token: c = RMSnorm(kv[:rank]) * norm_w and the rotated shared key part rope(kv[rank:]) go to
     cache row ``slots[t]`` (< 0: no write; ``cache`` [rows, rank + rot_dim]); every head's rotated
     query part ``q[t, h*head_stride + rot_off : +rot_dim]`` is rotated into the returned
-    [T, heads, rot_dim].  Angles are pos * inv_freq in f32, pairs interleaved."""
+    [T, heads, rot_dim].  Angles are pos * inv_freq in f32, pairs interleaved, cos and sin times ``mscale``."""
     T = kv.shape[0]
     R, Dr, H = rank, rot_dim, heads
     if N.use_native(kv):
         assert kv.dtype == cache.dtype == q.dtype
         q_rot = torch.empty((T, H, Dr), dtype=q.dtype, device=q.device)
         N.mcall("mx_latent_prep", N.ptr(_rows(kv)), kv.stride(0), N.ptr(norm_w), float(eps), N.ptr(inv_freq),
-                int(rot_dims), N.ptr(pos), N.ptr(slots), N.ptr(cache), N.ptr(_rows(q)), q.stride(0), head_stride,
+                int(rot_dims), float(mscale), N.ptr(pos), N.ptr(slots), N.ptr(cache), N.ptr(_rows(q)), q.stride(0), head_stride,
                 rot_off, N.ptr(q_rot), _dt(kv), T, H, R, Dr, N.stream())
         return q_rot
     kvf = kv.float()
     c = kvf[:, :R]
     c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
     ang = pos.float()[:, None] * inv_freq.float()[None, :rot_dims // 2]
-    kr = _rotate(kvf[:, R:R + Dr], ang, rot_dims)
+    kr = _rotate(kvf[:, R:R + Dr], ang, rot_dims, mscale)
     rows = torch.cat([c, kr], 1).to(cache.dtype)
     ok = slots >= 0
     cache.view(-1, R + Dr)[slots[ok].long()] = rows[ok]
     qr = torch.stack([q[:, h * head_stride + rot_off:h * head_stride + rot_off + Dr] for h in range(H)], 1).float()
-    return _rotate(qr, ang[:, None, :], rot_dims).to(q.dtype)
+    return _rotate(qr, ang[:, None, :], rot_dims, mscale).to(q.dtype)
+
+
+def _sink_softmax(sc: torch.Tensor, sink: Optional[torch.Tensor]) -> torch.Tensor:
+    """Softmax over the last axis of f32 scores [n, H, keys]; ``sink`` [H]: one more entry of the denominator."""
+    if sink is None:
+        return torch.softmax(sc, -1)
+    extra = sink.float()[None, :, None].expand(sc.shape[0], sc.shape[1], 1)
+    return torch.softmax(torch.cat([sc, extra], -1), -1)[..., :-1]
 
 
 def latent_attend(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: torch.Tensor,
                   bt: torch.Tensor, window: int, scale: float, max_len: int,
-                  gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  gate: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
+                  exact_weights: bool = False) -> torch.Tensor:
     """Windowed causal attention in the latent space.  ``q_lat`` [T, H, R], ``q_rot`` [T, H, Dr];
     cache rows [c | k_rot]; the query at position p sees the keys j of its own sequence with
     0 <= p - j < window; score = (q_lat . c_j + q_rot . k_rot_j) * scale, f32 softmax,
-    out[t, h] = sum_j p_j c_j, times sigmoid(gate[t, h]) when a gate [T, H] is given."""
+    out[t, h] = sum_j p_j c_j, times sigmoid(gate[t, h]) when a gate [T, H] is given.  ``sink`` (f32 [H]): the
+    softmax denominator of head h also holds exp(sink[h]).  ``exact_weights``: the bf16 kernel multiplies the
+    latents by the softmax weights as two bf16 terms instead of one (f32 kernels always use f32 weights)."""
     T, H, R = q_lat.shape
     Dr = q_rot.shape[2]
     S = cu.numel() - 1
+    if sink is not None and (sink.dtype != torch.float32 or sink.numel() != H):
+        raise ValueError("sink: one f32 value per query head")
     if N.use_native(q_lat):
         assert q_lat.is_contiguous() and q_rot.is_contiguous() and bt.is_contiguous()
         out = torch.empty((T, H, R), dtype=q_lat.dtype, device=q_lat.device)
@@ -404,8 +447,8 @@ def latent_attend(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor,
                 ws = torch.empty((T, H, nsplit, R + 2), dtype=torch.float32, device=q_lat.device)
         N.mcall("mx_latent_attend", N.ptr(q_lat), N.ptr(q_rot), N.ptr(cache), N.ptr(cu), N.ptr(pos), N.ptr(bt),
                 bt.shape[1], N.ptr(_rows(gate)) if gate is not None else None,
-                gate.stride(0) if gate is not None else 0, int(min(window, 1 << 30)), float(scale), N.ptr(out),
-                _dt(q_lat), S, int(max_len), H, R, Dr, nsplit, N.ptr(ws), N.stream())
+                gate.stride(0) if gate is not None else 0, N.ptr(sink), 1 if exact_weights else 0,
+                int(min(window, 1 << 30)), float(scale), N.ptr(out), _dt(q_lat), S, int(max_len), H, R, Dr, nsplit, N.ptr(ws), N.stream())
         return out
     out = torch.zeros((T, H, R), dtype=torch.float32)
     rows = cache.view(-1, R + Dr).float()
@@ -423,7 +466,7 @@ def latent_attend(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor,
         j = torch.arange(ctx)[None]
         vis = (j <= p) & (j > p - window)
         sc = sc.masked_fill(~vis[:, None, :], float("-inf"))
-        out[a:b] = torch.einsum("nhj,jr->nhr", torch.softmax(sc, -1), keys[:, :R])
+        out[a:b] = torch.einsum("nhj,jr->nhr", _sink_softmax(sc, sink), keys[:, :R])
     if gate is not None:
         out = out * torch.sigmoid(gate.float())[:, :, None]
     return out.to(q_lat.dtype)
@@ -780,26 +823,40 @@ def mingru_scan(zp: torch.Tensor, xp: torch.Tensor, gp: torch.Tensor, z_bias: Op
 # sliding-window attention with grouped key/value heads over a paged row cache
 # ----------------------------------------------------------------------------------------------
 def qk_norm_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, qw: Optional[torch.Tensor],
-                  kw: Optional[torch.Tensor], eps: float, slots: torch.Tensor, cache: torch.Tensor) -> torch.Tensor:
+                  kw: Optional[torch.Tensor], eps: float, slots: torch.Tensor, cache: torch.Tensor, dim: int = 0,
+                  freq: Optional[torch.Tensor] = None, pos: Optional[torch.Tensor] = None, layout: str = "half",
+                  mscale: float = 1.0) -> torch.Tensor:
     """Per token: RMS norm of the WHOLE query projection (all heads at once) times ``qw`` -> returned
     [T, nq]; the same for the key projection with ``kw``; the normed keys and the values go to cache
     row ``slots[t]`` as [k | v] (< 0: no write).  ``qw``/``kw`` None: no norm (without ``qw`` the returned
-    queries are ``q`` itself, a column slice: nothing is copied)."""
+    queries are ``q`` itself, a column slice: nothing is copied).  With ``freq`` (f32 [rot / 2]) the first ``rot``
+    entries of every head of ``dim`` entries are rotated after the norm by the angle pos * freq_i (f32), pairs as in
+    :func:`rope_heads`, cos and sin times ``mscale``."""
     T, nq = q.shape
     nk, nv = k.shape[1], v.shape[1]
     assert cache.shape[-1] == nk + nv
+    rot = 2 * freq.numel() if freq is not None else 0
+    if rot and (layout not in ("half", "pairs") or rot > dim or nq % dim or nk % dim or pos is None):
+        raise ValueError("qk_norm_write: whole heads of dim entries, rotated part <= dim, layout half | pairs")
     if N.use_native(q):
         assert q.dtype == k.dtype == v.dtype == cache.dtype
-        out = torch.empty((T, nq), dtype=q.dtype, device=q.device) if qw is not None else None
+        out = torch.empty((T, nq), dtype=q.dtype, device=q.device) if qw is not None or rot else None
         N.mcall("mx_qk_norm_write", N.ptr(_rows(q)), q.stride(0), N.ptr(_rows(k)), k.stride(0), N.ptr(_rows(v)), v.stride(0),
-                N.ptr(qw), N.ptr(kw), float(eps), N.ptr(slots), N.ptr(cache), N.ptr(out), _dt(q), T, nq, nk, nv, N.stream())
+                N.ptr(qw), N.ptr(kw), float(eps), int(dim), rot, 1 if layout == "half" else 0, N.ptr(freq), float(mscale),
+                N.ptr(pos), N.ptr(slots), N.ptr(cache), N.ptr(out), _dt(q), T, nq, nk, nv, N.stream())
         return out if out is not None else q
     rms = lambda t, w: (t.float() * torch.rsqrt(t.float().pow(2).mean(-1, keepdim=True) + eps) * w.float()  # noqa: E731
                         if w is not None else t.float())
-    rows = torch.cat([rms(k, kw), v.float()], 1).to(cache.dtype)
+    ang = pos.float()[:, None] * freq.float()[None, :] if rot else None
+
+    def done(t, w):
+        t = rms(t, w)
+        return _rotate_heads(t.reshape(T, -1, dim), ang, rot, layout == "half", mscale).reshape(T, -1) if rot else t
+
+    rows = torch.cat([done(k, kw), v.float()], 1).to(cache.dtype)
     ok = slots >= 0
     cache.view(-1, nk + nv)[slots[ok].long()] = rows[ok]
-    return rms(q, qw).to(q.dtype) if qw is not None else q
+    return done(q, qw).to(q.dtype) if qw is not None or rot else q
 
 
 def conv_heads(proj: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], q_norm: Optional[torch.Tensor],
@@ -858,11 +915,30 @@ def conv_heads(proj: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor
     return q.to(proj.dtype)
 
 
+def distance_buckets(rows: int, far: float) -> torch.Tensor:
+    """Row of a ``rows``-row bias table for every distance 0 .. L - 1 (int64; L - 1 is the first distance of the last
+    row, which every larger distance shares): distance n itself below rows/2, from there in logarithmic steps that
+    reach the last row before ``far``: rows/2 + floor(ln(n / (rows/2)) / ln(far / (rows/2)) * (rows - rows/2))."""
+    import math
+    half = rows // 2
+    if half < 1 or not far > half:
+        raise ValueError("distance buckets: at least two rows and far > rows / 2")
+    out, n = list(range(half)), half
+    while out[-1] < rows - 1:
+        r = math.log(n / half) / math.log(far / half) * (rows - half)
+        if abs(r - round(r)) < 1e-9:         # a step that falls on a whole distance is not left to rounding
+            r = round(r)
+        out.append(min(rows - 1, half + math.floor(r)))
+        n += 1
+    return torch.tensor(out, dtype=torch.int64)
+
+
 def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: torch.Tensor, bt: torch.Tensor,
                   window: int, scale: float, max_len: int, heads: int, kv_heads: int, dim: int, vdim: int,
                   gate: Optional[torch.Tensor] = None, chunked: bool = False, keep_first: int = 0,
                   head_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None,
-                  sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  sink: Optional[torch.Tensor] = None, rel: Optional[torch.Tensor] = None,
+                  softcap: float = 0.0) -> torch.Tensor:
     """Causal softmax attention of ``q`` [T, H*dim] over the cache rows [k: G*dim | v: G*vdim] of each
     segment's pages: the query at position p sees keys j with 0 <= p - j < window, or -- ``chunked`` --
     the keys j <= p with floor(j / window) == floor(p / window) (blocks of ``window`` positions counted
@@ -870,7 +946,9 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
     visible to every later query as well (at their true positions).  Query head h
     reads key/value head h // (H/G); score = q . k * scale, f32 softmax -- or, with ``head_bias`` (f32 [H]),
     no softmax: the weight of a visible key is sigmoid(score + head_bias[h]), not normalised over the keys.
-    ``slopes`` (f32 [H]): a distance bias, slopes[h] * (p - j) is taken off the scaled score.  ``sink`` (f32 [H],
+    ``softcap`` > 0: the scaled score becomes softcap * tanh(score / softcap) before any bias.  ``slopes`` (f32 [H]): a
+    distance bias, slopes[h] * (p - j) is taken off the score; ``rel`` (f32 [H, L]): another, rel[h, min(p - j, L - 1)]
+    is added to it.  ``sink`` (f32 [H],
     softmax only): the denominator of head h also holds exp(sink[h]).  Head h's output is multiplied by
     sigmoid(gate[t, h]) when a gate [T, H] is given, or element by element by sigmoid(gate) when the gate is
     [T, H*vdim].  Returns [T, H*vdim]."""
@@ -883,6 +961,8 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
             raise ValueError(f"{name}: one f32 value per query head")
     if sink is not None and head_bias is not None:
         raise ValueError("a sink belongs to the softmax denominator; sigmoid weights have none")
+    if rel is not None and (rel.dtype != torch.float32 or rel.dim() != 2 or rel.shape[0] != H or not rel.is_contiguous()):
+        raise ValueError("rel: a contiguous f32 table [heads, distances]")
     if gate is not None and gate.shape[1] not in (H, H * P):
         raise ValueError("gate: one value per head or per output element")
     gate_elem = gate is not None and P > 1 and gate.shape[1] == H * P
@@ -900,7 +980,8 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
         N.mcall("mx_window_attend", N.ptr(_rows(q)), q.stride(0), N.ptr(cache), N.ptr(cu), N.ptr(pos), N.ptr(bt), bt.shape[1],
                 N.ptr(_rows(gate)) if gate is not None else None, gate.stride(0) if gate is not None else 0,
                 1 if gate_elem else 0, int(min(window, 1 << 30)), 1 if chunked else 0, int(keep_first), N.ptr(head_bias),
-                N.ptr(slopes), N.ptr(sink), float(scale), N.ptr(out),
+                N.ptr(slopes), N.ptr(rel), rel.shape[1] if rel is not None else 0, float(softcap), N.ptr(sink), float(scale),
+                N.ptr(out),
                 _dt(q), S, int(max_len), H, G, D, P, nsplit, N.ptr(ws), N.stream())
         return out
     out = torch.zeros((T, H, P), dtype=torch.float32)
@@ -919,6 +1000,10 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
         sc = torch.einsum("nhd,jhd->nhj", q[a:b].float().view(-1, H, D), keys) * scale
         p = pos[a:b].long()[:, None]
         j = torch.arange(ctx)[None]
+        if softcap > 0:
+            sc = softcap * torch.tanh(sc / softcap)
+        if rel is not None:
+            sc = sc + rel[:, (p - j).clamp(0, rel.shape[1] - 1)].transpose(0, 1)
         if slopes is not None:
             sc = sc - slopes.float()[None, :, None] * (p - j).float()[:, None, :]
         vis = (j <= p) & (((j // window == p // window) if chunked else (j > p - window)) | (j < keep_first))
@@ -926,9 +1011,7 @@ def window_attend(q: torch.Tensor, cache: torch.Tensor, cu: torch.Tensor, pos: t
             wt = torch.sigmoid(sc + head_bias.float()[None, :, None]) * vis[:, None, :]
         else:
             sc = sc.masked_fill(~vis[:, None, :], float("-inf"))
-            if sink is not None:                # one more entry of the denominator, without a value
-                sc = torch.cat([sc, sink.float()[None, :, None].expand(sc.shape[0], H, 1)], -1)
-            wt = torch.softmax(sc, -1)[..., :ctx]
+            wt = _sink_softmax(sc, sink)
         out[a:b] = torch.einsum("nhj,jhp->nhp", wt, vals)
     if gate is not None:
         out = out * torch.sigmoid(gate.float()).view(T, H, P if gate_elem else 1)
@@ -1003,7 +1086,9 @@ def rope_freqs(dims: int, base: float, scaling: Optional[dict] = None, device=No
     ``scaling`` entry {factor, original, fast, slow} (YaRN): with turn(t) = dims ln(original / (2 pi t)) /
     (2 ln base), lo = max(floor(turn(fast)), 0), hi = min(ceil(turn(slow)), dims - 1) and
     ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1) the frequency is f_i / factor * ramp_i +
-    f_i (1 - ramp_i) and cos and sin are multiplied by 0.1 ln(factor) + 1.  A ``scaling`` entry with a factor
+    f_i (1 - ramp_i) and cos and sin are multiplied by 0.1 ln(factor) + 1.  With {factor, original, low, high}
+    (scaling by wavelength l = 2 pi / f): f is kept where l < original / high, divided by the factor where
+    l > original / low, and (1 - s) f / factor + s f with s = (original / l - low) / (high - low) between.  A ``scaling`` entry with a factor
     only is linear scaling: every f_i is divided by the factor (positions are stretched), cos and sin unscaled."""
     import math
     i = torch.arange(dims // 2, dtype=torch.float64)
@@ -1011,6 +1096,13 @@ def rope_freqs(dims: int, base: float, scaling: Optional[dict] = None, device=No
     m = 1.0
     if scaling and "original" not in scaling:      # linear scaling: every frequency divided by the factor
         f = f / float(scaling["factor"])
+    elif scaling and "high" in scaling:
+        factor, orig = float(scaling["factor"]), float(scaling["original"])
+        low, high = float(scaling["low"]), float(scaling["high"])
+        wave = 2 * math.pi / f
+        s = (orig / wave - low) / (high - low) if high != low else torch.zeros_like(f)
+        blend = (1 - s) * f / factor + s * f
+        f = torch.where(wave < orig / high, f, torch.where(wave > orig / low, f / factor, blend))
     elif scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
         turn = lambda t: dims * math.log(orig / (2 * math.pi * float(t))) / (2 * math.log(float(base)))  # noqa: E731
