@@ -88,11 +88,12 @@ def parse(argv=None):
                          "multi-GPU measurement")
     ap.add_argument("--json-out", default="")
     ap.add_argument("--model-throughput", default="", metavar="DESIGN",
-                    choices=["", "gezavik", "sigudra", "tukedra", "purozen", "fanotar"],
+                    choices=["", "gezavik", "sigudra", "tukedra", "purozen", "fanotar", "sepitar"],
                     help="instead of the serving workload: prefill and decode tokens/s of the named layered design at "
                          "a few layer sizes beside its closest relative of equal size (gezavik: a Llama twin; sigudra: "
                          "Gezavik; tukedra: Sigudra; purozen: a Sigudra with dense feed-forwards; fanotar: a "
-                         "Tukedra with attention layers only) (bench/model_throughput.py; one JSON "
+                         "Tukedra with attention layers only; sepitar: a Gezavik with attention layers only and a Fanotar "
+                         "with routed feed-forwards only) (bench/model_throughput.py; one JSON "
                          "line per model and workload)")
     from financial_chatbot_llm_amd.bench.model_throughput import add_arguments
     add_arguments(ap)

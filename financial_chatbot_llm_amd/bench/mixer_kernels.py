@@ -1,6 +1,6 @@
 """Times the sequence-mixer kernels (``ops.mixers``) at the layer shapes of a hybrid decoder.
 
-    python -m financial_chatbot_llm_amd.bench.mixer_kernels [--width 2048] [--design gezavik|sigudra|tukedra|purozen|fanotar]
+    python -m financial_chatbot_llm_amd.bench.mixer_kernels [--width 2048] [--design gezavik|sigudra|tukedra|purozen|fanotar|sepitar]
 
 Two step shapes: a prefill step of two 2048-token prompts and a decode step of 64 single rows at
 depth 1024.  Shapes follow ``models.gezavik.example_config(scale_up=True)``: Mamba-2 with inner =
@@ -20,6 +20,9 @@ wide as the model; position-free latent attention of rank 256; the gated residua
 ``--design fanotar``: that design's kernels at ``models.fanotar.example_config(scale_up=True)`` shapes (width / 128
 heads of 128 with 4 query heads per key/value head, 4 taps, window 1024 with distance bias, sink and elementwise
 gate; the elementwise norms around a sublayer; clamped units; routing over 32 experts, top 4).
+``--design sepitar``: that design's kernels at ``models.sepitar.example_config(scale_up=True)`` shapes (distance-biased
+windowed attention and soft-capped causal attention with width / 128 heads of 128 on a quarter of the key/value heads,
+latent attention of rank 256 with 32 rotated entries), each beside the same call without the design's options.
 """
 from __future__ import annotations
 
@@ -320,11 +323,97 @@ def fanotar(width: int) -> int:
     return 0
 
 
+def sepitar(width: int) -> int:
+    dev = "cuda"
+    H, D, P, window, B = max(width // 128, 2), 128, 128, 1024, 32
+    G, R, Dr, dn = max(H // 4, 1), 256, 32, 96
+    out = lambda **kw: print(json.dumps(kw), flush=True)  # noqa: E731
+    for name, lens, start, cu, pos, slot in _steps(dev):
+        S, T, ml = len(lens), sum(lens), max(lens)
+        pages = (start + ml + 63) // 64
+        bt = torch.arange(S * pages, dtype=torch.int32, device=dev).view(S, pages).contiguous()
+        slots = (bt[:, None, :].expand(S, ml, pages).reshape(-1, pages).gather(1, (pos // 64).long()[:, None])[:, 0] * 64
+                 + pos % 64).to(torch.int32)
+        cache = torch.randn(S * pages * 64, G * (D + P), device=dev).bfloat16()
+        nq, nk, nv = H * D, G * D, G * P
+        proj = torch.randn(T, nq + nk + nv + H * P, device=dev).bfloat16()
+        q, k, v, gate = proj[:, :nq], proj[:, nq:nq + nk], proj[:, nq + nk:nq + nk + nv], proj[:, nq + nk + nv:]
+        qw, kw = torch.ones(nq, device=dev), torch.ones(nk, device=dev)
+        freq, ms = mx.rope_freqs(D, 5e5, {"factor": 8.0, "high": 4.0, "low": 1.0, "original": 8192}, device=dev)
+        byts = T * (2 * nq + 2 * nk + 2 * nv) * 2
+        us = _time(lambda: mx.qk_norm_write(q, k, v, qw, kw, 1e-5, slots, cache, dim=D, freq=freq, pos=pos, mscale=ms))
+        out(shape=name, kernel="qk_norm_write + rotation", us=round(us, 1), TB_per_s=round(byts / us / 1e6, 2))
+        us = _time(lambda: mx.qk_norm_write(q, k, v, qw, kw, 1e-5, slots, cache))
+        out(shape=name, kernel="qk_norm_write (norms only)", us=round(us, 1), TB_per_s=round(byts / us / 1e6, 2))
+        us = _time(lambda: mx.qk_norm_write(q, k, v, None, None, 1e-5, slots, cache))
+        out(shape=name, kernel="qk_norm_write (cache write only)", us=round(us, 1),
+            TB_per_s=round(T * (nk + nv) * 4 / us / 1e6, 2))
+        us = _time(lambda: mx.rope_heads(q, k, H, G, D, freq, pos, "half", ms, norm_eps=1e-5, k_out=cache, slots=slots, v=v))
+        out(shape=name, kernel="rope_heads + cache write (same bytes)", us=round(us, 1), TB_per_s=round(byts / us / 1e6, 2))
+        qn = mx.qk_norm_write(q, k, v, qw, kw, 1e-5, slots, cache, dim=D, freq=freq, pos=pos, mscale=ms)
+        rel = torch.randn(B, H, device=dev)[mx.distance_buckets(B, 1024.0).to(dev)].t().contiguous()
+        sink, slopes = torch.zeros(H, device=dev), torch.full((H,), 0.05, device=dev)
+        gh = gate[:, :H]
+        for label, win, kwargs in (("distance table + elementwise gate, window", window, dict(gate=gate, rel=rel)),
+                                   ("slopes + sink + elementwise gate, window", window, dict(gate=gate, slopes=slopes, sink=sink)),
+                                   ("plain, window", window, {}),
+                                   ("soft cap + sink + head gate, causal", 1 << 30, dict(gate=gh, sink=sink, softcap=30.0)),
+                                   ("plain, causal", 1 << 30, {})):
+            us = _time(lambda: mx.window_attend(qn, cache, cu, pos, bt, win, D ** -0.5, ml, H, G, D, P, **kwargs), 5)
+            pairs = sum(min(p + 1, win) for n in lens for p in range(start, start + n))
+            out(shape=name, kernel=f"window_attend {label}", us=round(us, 1),
+                bf16_TFLOP_per_s=round(pairs * H * 2 * (D + P) / us / 1e6, 1),
+                cache_TB_per_s=round(S * min(start + ml, win + ml) * G * (D + P) * 2 / us / 1e6, 3))
+        lcache = torch.randn(S * pages * 64, R + Dr, device=dev).bfloat16()
+        kv = torch.randn(T, R + Dr, device=dev).bfloat16()
+        qq = torch.randn(T, H * (dn + Dr), device=dev).bfloat16()
+        nw = torch.ones(R, device=dev)
+        lf, lm = mx.rope_freqs(Dr, 1e4, {"factor": 4.0, "fast": 32.0, "original": 4096, "slow": 1.0}, device=dev)
+        prep = lambda: mx.latent_prep(kv, nw, 1e-5, lf, Dr, pos, slots, lcache, qq, H, dn + Dr, dn, R, Dr, lm)  # noqa: E731
+        us = _time(prep)
+        out(shape=name, kernel="latent_prep", us=round(us, 1), TB_per_s=round(T * (2 * (R + Dr) + 2 * H * Dr) * 2 / us / 1e6, 2))
+        ql, qr = torch.randn(T, H, R, device=dev).bfloat16() * .1, prep()
+        pairs = sum(min(p + 1, window) for n in lens for p in range(start, start + n))
+        for label, kwargs in (("sink, two-term weights", dict(sink=sink, exact_weights=True)),
+                              ("head gate, one-term weights", dict(gate=gh))):
+            us = _time(lambda: mx.latent_attend(ql, qr, lcache, cu, pos, bt, window, 0.1, ml, **kwargs), 5)
+            out(shape=name, kernel=f"latent_attend {label}", us=round(us, 1),
+                bf16_TFLOP_per_s=round(pairs * H * 2 * (2 * R + Dr) / us / 1e6, 1),
+                cache_TB_per_s=round(S * min(start + ml, window + ml) * (R + Dr) * 2 / us / 1e6, 3))
+        x = torch.randn(T, width, device=dev)
+        a, b = torch.randn(T, width, device=dev).bfloat16(), torch.randn(T, width, device=dev).bfloat16()
+        w = torch.ones(width, device=dev)
+        table = torch.randn(32768, width, device=dev).bfloat16()
+        ids = torch.randint(0, 32768, (T,), dtype=torch.int32, device=dev)
+        us = _time(lambda: mx.residual_norm(x, w, 1e-5, a, b))
+        out(shape=name, kernel="residual_norm two sublayers", us=round(us, 1), TB_per_s=round(T * width * 14 / us / 1e6, 2))
+        us = _time(lambda: mx.residual_norm(x, w, 1e-5, a, b, ids=ids, table=table))
+        out(shape=name, kernel="residual_norm two sublayers + embedding row", us=round(us, 1),
+            TB_per_s=round(T * width * 16 / us / 1e6, 2))
+        us = _time(lambda: mx.embed_norm(ids, table, w, 1e-5))
+        out(shape=name, kernel="embed_norm", us=round(us, 1), TB_per_s=round(T * width * 8 / us / 1e6, 2))
+        ff = width // 2
+        gu = torch.randn(T * 4, 2 * ff, device=dev).bfloat16()
+        us = _time(lambda: mx.glu_clamp(gu[:, :ff], gu[:, ff:], 7.0, 1.702))
+        out(shape=name, kernel="glu_clamp over the expert buckets", us=round(us, 1), TB_per_s=round(T * 4 * ff * 6 / us / 1e6, 2))
+        z = torch.randn(T, 32, device=dev)
+        us = _time(lambda: mx.route_scores(z, 4, "softmax_top"))
+        out(shape=name, kernel="route_scores softmax_top", us=round(us, 1))
+        ys = torch.randn(T * 4, width, device=dev).bfloat16()
+        wt, idx = mx.route_scores(z, 4, "softmax_top")
+        ps = torch.arange(T * 4, dtype=torch.int32, device=dev).view(T, 4)
+        us = _time(lambda: mx.moe_combine(ys, ps, idx, wt, a, b, 32))
+        out(shape=name, kernel="moe_combine top 4 + shared", us=round(us, 1), TB_per_s=round(T * width * 12 / us / 1e6, 2))
+    return 0
+
+
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--width", type=int, default=2048)
-    ap.add_argument("--design", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen", "fanotar"])
+    ap.add_argument("--design", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen", "fanotar", "sepitar"])
     a = ap.parse_args(argv)
+    if a.design == "sepitar":
+        return sepitar(a.width)
     if a.design == "fanotar":
         return fanotar(a.width)
     if a.design == "purozen":

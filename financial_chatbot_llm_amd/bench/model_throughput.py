@@ -5,6 +5,7 @@
     python bench.py --model-throughput tukedra          # beside Sigudra, its closest relative here
     python bench.py --model-throughput purozen          # beside a dense-feed-forward Sigudra of equal size
     python bench.py --model-throughput fanotar          # beside an attention-only Tukedra of equal size
+    python bench.py --model-throughput sepitar          # beside an attention-only Gezavik and an all-routed Fanotar
     python -m financial_chatbot_llm_amd.bench.model_throughput --mt-only gezavik-w2048
 
 For each width a Gezavik model (random weights, 8 layers: latent attention and Mamba-2 mixers, dense
@@ -127,6 +128,25 @@ def register_fanotar(width: int, vocab: int = 32768) -> List[str]:
     return [name, twin]
 
 
+def register_sepitar(width: int, vocab: int = 32768) -> List[str]:
+    """Register ``sepitar-w<width>`` (6 layers ``LRCLRC`` of which the second and third run twice, 8 layer runs: latent
+    attention, distance-biased attention, soft-capped attention; every layer with routed clamped units and a shared
+    expert), ``gezavik-att-w<width>``, the Gezavik model of the same width, vocabulary and 8 layers with latent
+    attention and routed feed-forwards only (parallel blocks as well), and ``fanotar-moe-w<width>``, the Fanotar model
+    of 8 layers with routed feed-forwards only (windowed attention, expert shapes as here); returns the three names."""
+    from ..models.configs import REGISTRY, layered_config
+    from ..models.fanotar import example_config as fanotar_config
+    from ..models.gezavik import example_config as gezavik_config
+    from ..models.sepitar import example_config
+    names = [f"sepitar-w{width}", f"gezavik-att-w{width}", f"fanotar-moe-w{width}"]
+    gez = gezavik_config(width=width, vocab=vocab, heads=max(width // 128, 2), pattern="A" * 8, scale_up=True)
+    configs = (example_config(width=width, vocab=vocab, pattern="LRCLRC", scale_up=True, loop=(1, 3, 2)), gez,
+               fanotar_config(width=width, vocab=vocab, pattern="E" * 8, scale_up=True))
+    for name, c in zip(names, configs):
+        REGISTRY[name] = layered_config(c, name)
+    return names
+
+
 def _tokens(n: int, vocab: int, seed: int) -> List[int]:
     g = torch.Generator().manual_seed(seed)
     return torch.randint(5, vocab - 300, (n,), generator=g).tolist()
@@ -199,7 +219,7 @@ def run(a) -> int:
     design = getattr(a, "model_throughput", "") or "gezavik"
     for w in (int(x) for x in a.mt_widths.split(",") if x):
         names += {"sigudra": register_sigudra, "tukedra": register_tukedra, "purozen": register_purozen,
-                  "fanotar": register_fanotar}.get(design, register)(w)
+                  "fanotar": register_fanotar, "sepitar": register_sepitar}.get(design, register)(w)
     if a.mt_only:
         names = [n for n in names if n == a.mt_only]
     for n in names:
@@ -210,7 +230,7 @@ def run(a) -> int:
 
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--model-throughput", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen", "fanotar"])
+    ap.add_argument("--model-throughput", default="gezavik", choices=["gezavik", "sigudra", "tukedra", "purozen", "fanotar", "sepitar"])
     add_arguments(ap)
     return run(ap.parse_args(argv))
 

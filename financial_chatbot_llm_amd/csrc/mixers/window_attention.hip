@@ -159,7 +159,8 @@ __global__ void qk_norm_rope_write_kernel(const T* __restrict__ q, long sq, cons
   T* dst = cache + (long)slot * (nk + nv);
   turn(kr, kw, ck, dst, nk);
   const T* vr = v + t * sv;
-  for (int i = threadIdx.x; i < nv; i += blockDim.x) dst[nk + i] = vr[i];
+  for (int i = threadIdx.x; i < nv / V; i += blockDim.x)
+    *reinterpret_cast<vec*>(dst + nk + (long)i * V) = *reinterpret_cast<const vec*>(vr + (long)i * V);
 }
 
 // Work layout: a block owns QT consecutive rows of one segment and HB query heads of ONE key/value
@@ -326,8 +327,11 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 constexpr int MKT = 32;             // keys per tile
 constexpr int MLDV = MKT + 8;       // row stride of the transposed value tile
 
-template <int KSM, int NTM>         // up to 32*KSM key dims, 16*NTM value dims
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2)))
+// up to 32*KSM key dims, 16*NTM value dims; CAP: soft-capped scores, REL: distance table (a form of its own each, so
+// that the plain walk's inner loop stays free of branches; these forms take no sigmoid weights, REL no slopes and no
+// kept first tokens)
+template <int KSM, int NTM, bool CAP, bool REL>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(KSM <= 4 ? 4 : 2)))
 window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __restrict__ cache,
                           const int* __restrict__ cu, const int* __restrict__ pos, const int* __restrict__ bt, int btw,
                           const bf16* __restrict__ gate, long sgate, int gate_elem, int window, int chunked, int keep,
@@ -367,7 +371,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
   const int pq = qok ? pos[row] : -1;
   const int pq_lo = qok ? first_key(pq, window, chunked) : 0;
   const bool wave_live = 16 * wave < nq * nh;
-  const bool sigm = hbias != nullptr;
+  const bool sigm = !CAP && !REL && hbias != nullptr;
   const float hb = (sigm && qok) ? hbias[h] : 0.f;
   const float slp = (slope != nullptr && qok) ? slope[h] : 0.f;     // distance bias: score + slp * (j - p)
 
@@ -393,7 +397,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
   }
 
   const int first_tile = lo / MKT;
-  const int nsink = min((keep + MKT - 1) / MKT, first_tile);
+  const int nsink = REL ? 0 : min((keep + MKT - 1) / MKT, first_tile);
   int t_begin = 0, t_end = nsink + p_last / MKT - first_tile;     // walk indices, inclusive
   if (nsplit > 1) {
     const int per = (t_end + nsplit) / nsplit;                    // ceil((t_end + 1) / nsplit)
@@ -406,10 +410,10 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
   float* rel_lds = reinterpret_cast<float*>(vt_lds + (size_t)NT * 16 * MLDV);
   int rel_off = 0;
   bool rel_tab = false;
-  if (rel != nullptr && t_begin <= t_end) {
+  if (REL && t_begin <= t_end) {
     const int kb = walk_k0(t_begin, nsink, first_tile, MKT);
     const int span = (p_last - p_first) + (t_end - t_begin + 1) * MKT;
-    rel_tab = ldr > 0 && nsink == 0 && span <= ldr;
+    rel_tab = ldr > 0 && span <= ldr;
     if (rel_tab) {
       const int far = p_last - kb;
       for (int e = threadIdx.x; e < nh * span; e += 256) {
@@ -419,7 +423,7 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
       rel_off = hh * ldr + far - max(pq, p_first) + 4 * g;      // + the key's position: its entry
     }
   }
-  const float cap_k = cap > 0.f ? 2.885390081777927f * scale / cap : 0.f;
+  const float cap_k = CAP ? 2.885390081777927f * scale / cap : 0.f;
   // staging, 16-byte path (D, P multiples of 8): a work item is a pair of keys x 8 dims of the key
   // part or of the value part -- two row loads; key pieces go to the key tile as two 16-byte stores,
   // value pieces to the transposed value tile as eight 4-byte stores (one key pair each).  The next
@@ -498,27 +502,24 @@ window_attend_mfma_kernel(const bf16* __restrict__ q, long sq, const bf16* __res
 #pragma unroll
       for (int ks = 0; ks < KSM; ++ks)
         if (ks < KS) st[kh] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kr + 32 * ks), qf[ks], st[kh], 0, 0, 0);
-      if (cap > 0.f) {
+      float add[4] = {0.f, 0.f, 0.f, 0.f};
+      if (REL) {
+        if (rel_tab) {
+          const float* rt = rel_lds + rel_off + k0 + 16 * kh;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) sc[kh][i] = soft_cap(st[kh][i], cap_k, cap);
-      } else {
+          for (int i = 0; i < 4; ++i) add[i] = rt[i];
+        } else {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) sc[kh][i] = st[kh][i] * scale;
-      }
-      if (rel_tab) {
-        const float* rt = rel_lds + rel_off + k0 + 16 * kh;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) sc[kh][i] += rt[i];
-      } else if (rel != nullptr) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          sc[kh][i] += rel[(long)h * rel_len + min(max(pq - (k0 + 16 * kh + 4 * g + i), 0), rel_len - 1)];
+          for (int i = 0; i < 4; ++i)
+            add[i] = rel[(long)h * rel_len + min(max(pq - (k0 + 16 * kh + 4 * g + i), 0), rel_len - 1)];
+        }
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int j = k0 + 16 * kh + 4 * g + i;
-        const bool vis = j <= pq && (j >= pq_lo || j < keep);
-        sc[kh][i] = vis ? sc[kh][i] + slp * (dist0 + (float)(16 * kh + i)) : -INFINITY;
+        const bool vis = j <= pq && (j >= pq_lo || (!REL && j < keep));
+        const float s = CAP ? soft_cap(st[kh][i], cap_k, cap) : st[kh][i] * scale;
+        sc[kh][i] = vis ? (REL ? s + add[i] : s + slp * (dist0 + (float)(16 * kh + i))) : -INFINITY;
         tmax = fmaxf(tmax, sc[kh][i]);
       }
     }
@@ -677,8 +678,8 @@ MX_API int mx_qk_norm_write(const void* q, long sq, const void* k, long sk, cons
       return (int)hipErrorInvalidValue;
     const size_t lds = (size_t)rot * sizeof(float);
     const int V = dt == 1 ? 4 : 8;
-    const bool vec = half && (rot / 2) % V == 0 && D % V == 0 && sq % V == 0 && sk % V == 0 && (nk + nv) % V == 0 &&
-                     ((size_t)q | (size_t)k | (size_t)cache | (size_t)qout) % 16 == 0;
+    const bool vec = half && (rot / 2) % V == 0 && D % V == 0 && sq % V == 0 && sk % V == 0 && sv % V == 0 &&
+                     nv % V == 0 && ((size_t)q | (size_t)k | (size_t)v | (size_t)cache | (size_t)qout) % 16 == 0;
 #define QK_ROPE_LAUNCH(TT, VV)                                                                                      \
   qk_norm_rope_write_kernel<TT, VV><<<T, 256, lds, st>>>((const TT*)q, sq, (const TT*)k, sk, (const TT*)v, sv, qw, kw, \
                                                          eps, D, rot, half, freq, mscale, pos, slots, (TT*)cache,    \
@@ -720,7 +721,9 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
   // 2: gate rows that 8-byte accesses may read (bf16)
   const int ge = !gate_elem ? 0 : (P % 4 == 0 && sgate % 4 == 0 && (size_t)gate % 8 == 0 ? 2 : 1);
   const int rep = H / G;
-  if (dt == 0 && D <= 256 && P <= 256 && wa_use_mfma()) {
+  const bool forms = (cap <= 0.f || head_bias == nullptr) &&
+                     (rel == nullptr || (head_bias == nullptr && slope == nullptr && keep == 0));
+  if (dt == 0 && D <= 256 && P <= 256 && forms && wa_use_mfma()) {
     // matrix-core form: 64 (row, head) pairs of one key/value head per block
     const int HB = rep < 64 ? rep : 64;
     const int QT = max_len == 1 ? 1 : (64 / HB > 0 ? 64 / HB : 1);
@@ -728,7 +731,7 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
     size_t lds = ((size_t)MKT * (KS * 32 + 8) + (size_t)NT * 16 * MLDV) * sizeof(bf16);
     // distance table: every distance a block can meet, rows apart by 16 banks; only where 64 KB hold it
     int ldr = 0;
-    if (rel != nullptr && keep == 0 && window <= 16384) {
+    if (rel != nullptr && window <= 16384) {
       const int need = window + 2 * QT + 64;
       ldr = (need + 47) / 64 * 64 + 16;
       if (lds + (size_t)HB * ldr * sizeof(float) <= 64 * 1024) lds += (size_t)HB * ldr * sizeof(float);
@@ -736,14 +739,21 @@ MX_API int mx_window_attend(const void* q, long sq, const void* cache, const int
     }
     if (max_len != 1 || ws == nullptr || nsplit < 1) nsplit = 1;
     dim3 grid(nsplit > 1 ? nsplit : (max_len + QT - 1) / QT, G * ((rep + HB - 1) / HB), S);
-    if (D <= 128 && P <= 128)
-      window_attend_mfma_kernel<4, 8><<<grid, 256, lds, st>>>(
-          (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked,
-          keep, head_bias, slope, rel, rel_len, ldr, cap, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
-    else
-      window_attend_mfma_kernel<8, 16><<<grid, 256, lds, st>>>(
-          (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked,
-          keep, head_bias, slope, rel, rel_len, ldr, cap, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws);
+#define WINDOW_LAUNCH(KSM, NTM, CAP, REL)                                                                             \
+  window_attend_mfma_kernel<KSM, NTM, CAP, REL><<<grid, 256, lds, st>>>(                                              \
+      (const bf16*)q, sq, (const bf16*)cache, cu, pos, bt, btw, (const bf16*)gate, sgate, ge, window, chunked, keep,  \
+      head_bias, slope, rel, rel_len, ldr, cap, sink, scale, (bf16*)out, H, G, D, P, QT, HB, nsplit, ws)
+#define WINDOW_FORM(KSM, NTM)                                      \
+  do {                                                             \
+    if (cap > 0.f && rel != nullptr) WINDOW_LAUNCH(KSM, NTM, true, true);   \
+    else if (cap > 0.f) WINDOW_LAUNCH(KSM, NTM, true, false);      \
+    else if (rel != nullptr) WINDOW_LAUNCH(KSM, NTM, false, true); \
+    else WINDOW_LAUNCH(KSM, NTM, false, false);                    \
+  } while (0)
+    if (D <= 128 && P <= 128) WINDOW_FORM(4, 8);
+    else WINDOW_FORM(8, 16);
+#undef WINDOW_FORM
+#undef WINDOW_LAUNCH
     if (nsplit > 1) {
       dim3 g2(S, H);           // single-row segments: row index == segment index
       window_merge_kernel<<<g2, P >= 128 ? 128 : 64, 0, st>>>(ws, (const bf16*)gate, sgate, ge, sink, (bf16*)out, H, P,

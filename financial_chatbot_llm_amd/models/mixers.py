@@ -1210,12 +1210,13 @@ class RelBiasAttentionMixer(_GroupedAttention):
     def __init__(self, spec: Dict, width: int, eps: float):
         super().__init__(spec, width, eps)
         self.far = float(spec["bias_max"])
+        self.buckets = int(spec["buckets"]) if spec.get("buckets") else None      # None: the tensor gives it
         self.in_rows = self.nq + self.nk + self.nv + self.no
 
     def shapes(self) -> Dict[str, tuple]:
         W = self.width
         return {"q": (self.nq, W), "q.b": (self.nq,), "k": (self.nk, W), "k.b": (self.nk,), "v": (self.nv, W),
-                "v.b": (self.nv,), "rel": (None, self.H), "g": (self.no, W), "o": (W, self.no), "o.b": (W,)}
+                "v.b": (self.nv,), "rel": (self.buckets, self.H), "g": (self.no, W), "o": (W, self.no), "o.b": (W,)}
 
     def load(self, get: Getter, dtype) -> torch.Tensor:
         self.o, self.o_b = get("o").to(dtype).contiguous(), get("o.b").to(dtype).contiguous()

@@ -47,7 +47,7 @@ def example_config(width: int = 160, vocab: int = 736, pattern: str = "LRC", sca
         lat = {"dim": 96, "heads": H, "kv_rank": 256, "mask": {"size": 1024}, "q_rank": 768,
                "rot": {"base": 10000.0, "dims": 32, "scaling": {"factor": 4.0, "fast": 32.0, "original": 4096, "slow": 1.0}},
                "rot_dim": 32, "scale": 128 ** -0.5, "vdim": 96}
-        rel = {"bias_max": 1024, "dim": 128, "heads": H, "kv_heads": G, "mask": {"size": 1024}, "scale": 128 ** -0.5,
+        rel = {"bias_max": 1024, "buckets": 32, "dim": 128, "heads": H, "kv_heads": G, "mask": {"size": 1024}, "scale": 128 ** -0.5,
                "vdim": 128}
         cap = {"dim": 128, "heads": H, "kv_heads": G, "rot": {"base": 500000.0, "dims": 128, "scaling": {
             "factor": 8.0, "high": 4.0, "low": 1.0, "original": 8192}}, "scale": 128 ** -0.5, "softcap": 30.0, "vdim": 128}
@@ -57,7 +57,7 @@ def example_config(width: int = 160, vocab: int = 736, pattern: str = "LRC", sca
         lat = {"dim": 24, "heads": 3, "kv_rank": 40, "mask": {"size": 21}, "q_rank": 56,
                "rot": {"base": 10000.0, "dims": 8, "scaling": {"factor": 3.0, "fast": 8.0, "original": 128, "slow": 0.5}},
                "rot_dim": 8, "scale": 0.2, "vdim": 20}
-        rel = {"bias_max": 30, "dim": 24, "heads": 6, "kv_heads": 2, "mask": {"size": 37}, "scale": 0.25, "vdim": 20}
+        rel = {"bias_max": 30, "buckets": 12, "dim": 24, "heads": 6, "kv_heads": 2, "mask": {"size": 37}, "scale": 0.25, "vdim": 20}
         cap = {"dim": 32, "heads": 4, "kv_heads": 2, "rot": {"base": 1000.0, "dims": 24, "scaling": {
             "factor": 5.0, "high": 6.0, "low": 1.5, "original": 96}}, "scale": 0.3, "softcap": 4.0, "vdim": 28}
         moe = {"expert": {"ff": 40, "limit": 1.2}, "kind": "moe", "router": {"experts": 7, "top": 3},
