@@ -64,13 +64,13 @@ def _run(cmd):
     return r.stdout
 
 
-def build_mixers(jobs: int = 8, verbose: bool = False) -> str:
+def build_mixers(jobs: int = 8, verbose: bool = False, force: bool = False) -> str:
     """``csrc/mixers`` -> ``libpenny_mixers.so`` (a few seconds)."""
-    return build_kernels(jobs, verbose, src_dir=MDIR, lib=MIXER_LIB, bdir=BUILD + "_mixers")
+    return build_kernels(jobs, verbose, src_dir=MDIR, lib=MIXER_LIB, bdir=BUILD + "_mixers", force=force)
 
 
 def build_kernels(jobs: int = 8, verbose: bool = False, debug: bool = False, src_dir: str = KDIR,
-                  lib: str = "", bdir: str = "", flags=None) -> str:
+                  lib: str = "", bdir: str = "", flags=None, force: bool = False) -> str:
     bdir = bdir or BUILD + ("_debug" if debug else "")
     lib = lib or kernel_lib(debug)
     flags = flags or (HIP_FLAGS_DEBUG if debug else HIP_FLAGS)
@@ -83,7 +83,7 @@ def build_kernels(jobs: int = 8, verbose: bool = False, debug: bool = False, src
     for s in srcs:
         o = os.path.join(bdir, os.path.basename(s)[:-4] + ".o")
         objs.append(o)
-        if _newer([s] + headers, o):
+        if force or _newer([s] + headers, o):
             todo.append((s, o))
 
     def one(so):
@@ -107,14 +107,14 @@ def runtime_lib_path() -> str:
     return os.path.join(PKG, "_penny_runtime" + suffix)
 
 
-def build_runtime(verbose: bool = False) -> str:
+def build_runtime(verbose: bool = False, force: bool = False) -> str:
     import pybind11
     srcs = sorted(glob.glob(os.path.join(RDIR, "*.cpp")))
     headers = glob.glob(os.path.join(RDIR, "*.h"))
     out = runtime_lib_path()
     if not srcs:
         return ""
-    if _newer(srcs + headers, out):
+    if force or _newer(srcs + headers, out):
         if verbose:
             print("[g++] runtime", flush=True)
         inc = [pybind11.get_include(), sysconfig.get_paths()["include"]]
@@ -125,12 +125,13 @@ def build_runtime(verbose: bool = False) -> str:
     return out
 
 
-def build_all(jobs: int = 8, verbose: bool = False, debug: bool = False) -> None:
-    build_kernels(jobs=jobs, verbose=verbose)
-    build_mixers(jobs=jobs, verbose=verbose)
+def build_all(jobs: int = 8, verbose: bool = False, debug: bool = False, force: bool = False) -> None:
+    """``force``: compile every source whatever the age of what is built."""
+    build_kernels(jobs=jobs, verbose=verbose, force=force)
+    build_mixers(jobs=jobs, verbose=verbose, force=force)
     if debug:
-        build_kernels(jobs=jobs, verbose=verbose, debug=True)
-    build_runtime(verbose=verbose)
+        build_kernels(jobs=jobs, verbose=verbose, debug=True, force=force)
+    build_runtime(verbose=verbose, force=force)
 
 
 def clean() -> None:
